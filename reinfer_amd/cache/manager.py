@@ -29,18 +29,21 @@ class CacheGroupSpec:
     """Layers (run-order entries) that share block tables. ``window`` 0: all keys."""
     window: int
     entries: Tuple[int, ...]
+    keep: int = 0           # a window's first tokens that stay in sight: their blocks are never given back before the end
 
 
-def plan_groups(windows: Sequence[Optional[int]]) -> List[CacheGroupSpec]:
+def plan_groups(windows: Sequence[Optional[int]], keeps: Optional[Sequence[int]] = None) -> List[CacheGroupSpec]:
     """Group run-order entries by what they keep.
 
     ``windows[i]`` is None for an entry without keys of its own (it reads
     another entry's cache, or keeps fixed-size state), 0 for all keys, W > 0 for
-    a window. Entries with equal needs share a group.
+    a window; ``keeps[i]`` is how many first tokens such a window keeps in sight
+    (none given: 0). Entries with equal needs share a group.
     """
-    by: Dict[int, List[int]] = {}
+    by: Dict[Tuple[int, int], List[int]] = {}
     for i, w in enumerate(windows):
         if w is None:
             continue
-        by.setdefault(int(w), []).append(i)
-    return [CacheGroupSpec(window=w, entries=tuple(es)) for w, es in sorted(by.items())]
+        keep = int(keeps[i]) if keeps is not None and w else 0
+        by.setdefault((int(w), keep), []).append(i)
+    return [CacheGroupSpec(window=w, entries=tuple(es), keep=k) for (w, k), es in sorted(by.items())]

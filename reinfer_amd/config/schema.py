@@ -94,6 +94,7 @@ class NormSpec:
     offset: float = 0.0  # the stored weight lies around zero: the factor is offset + w (1.0 for "one plus w")
     groups: int = 1      # the row is normed in this many equal consecutive parts, each over its own root mean square
     scalar: bool = False # the stored weight is one number that multiplies every coordinate
+    factor: float = 1.0  # the weight is multiplied by this (a constant on whatever a linear map makes of the norm)
 
 
 @dataclass(frozen=True)
@@ -133,6 +134,9 @@ class MixerSpec:
     rotate_values: bool = False     # a value is turned by its own position over its whole size, a head's result back by the query's
     out_gate: bool = False          # the concatenated heads times sigmoid(W_g h), element by element, before the output projection
     kv_shared: bool = False         # the mixer has no key and value tensors: it reads another run entry's cache
+    keep_first: int = 0             # with a window: a request's first tokens that stay in sight
+    values_are_keys: bool = False   # no value tensors: a value is the key as projected, before norm and rotation
+    out_bias: bool = False          # the output projection has a bias
 
     def option(self, name: str, default: Any = None) -> Any:
         return dict(self.extra).get(name, default)
@@ -213,14 +217,46 @@ class MatrixMemorySpec:
 @dataclass(frozen=True)
 class DecayMemorySpec:
     """A matrix state a head that fades by a constant a head (``MixerSpec.params`` of the "decay_memory" mixer):
-    S <- decays[h] * S + k v^T, o = S^T q, with ``heads`` heads of ``key_dim`` x ``value_dim`` and silu on q, k and
-    v; the concatenated read-outs are RMS-normed together (``norm_eps``), times a plain weight and a sigmoid
-    gate."""
+    S <- decays[h] * S + k v^T, o = S^T q, with ``heads`` heads of ``key_dim`` x ``value_dim``. ``act`` "silu": silu on
+    q, k and v; "none": as projected, q and k turned by ``position`` (half-split pairs), k times ``k_scale``. The read-outs
+    are RMS-normed (``norm_eps``) all together or, with ``head_norm``, head by head, times a plain weight of that size
+    (``norm_weight`` False: none) and the ``gate`` ("sigmoid" or "silu") of a projection."""
     heads: int
     key_dim: int
     value_dim: int
     decays: Tuple[float, ...]
     norm_eps: float
+    act: str = "silu"
+    position: PositionSpec = PositionSpec("none")
+    k_scale: float = 1.0
+    head_norm: bool = False
+    norm_weight: bool = True
+    gate: str = "sigmoid"
+
+
+@dataclass(frozen=True)
+class GatedLinearSpec:
+    """A matrix state a head whose rows fade by a factor a key channel and token (``MixerSpec.params`` of the
+    "gated_linear" mixer): alpha = sigmoid(z)^(1 / tau) with z from a low-rank pair of ``rank`` and a bias,
+    S <- diag(alpha) S + k v^T, o = S^T q, q times ``q_scale``; ``norm_eps`` of the per-head norm of the read-out, whose
+    weight the heads share; a silu gate."""
+    heads: int
+    key_dim: int
+    value_dim: int
+    rank: int
+    tau: float
+    norm_eps: float
+    q_scale: float = 1.0
+
+
+@dataclass(frozen=True)
+class HyperSpec:
+    """Several residual streams (``BlockSpec.params`` of the "hyper" arrangement): ``streams`` copies of the stream, of
+    which each sublayer reads a weighted sum and which its result changes all at once by a [from, to] matrix and a factor
+    a stream. Tensors ``<name>.in``, ``<name>.out`` [streams] and ``<name>.mix`` [streams, streams], ``names`` for the mixer
+    and the feed-forward."""
+    streams: int
+    names: Tuple[str, str] = ("hc1", "hc2")
 
 
 @dataclass(frozen=True)
@@ -370,8 +406,17 @@ class ModelSpec:
     logit_softcap: float = 0.0
     # the embedding rows are multiplied by this on their way into the stream (a tied head uses the table as it is)
     embed_scale: float = 1.0
+    # copies of the residual stream that the blocks read and mix (0: one stream, the usual sum); every block is then of
+    # an arrangement for several streams
+    streams: int = 0
 
     def __post_init__(self):
+        if self.streams:
+            for b in self.blocks:
+                if getattr(b.params, "streams", None) != self.streams:
+                    raise ConfigError("streams", f"block {b.prefix!r} is not made for {self.streams} streams")
+            if any(e.before is not None for e in self.run_order):
+                raise ConfigError("streams", "nothing is added between the layers of a model of several streams")
         for i, e in enumerate(self.run_order):
             if not 0 <= e.block < len(self.blocks):
                 raise ConfigError("run_order", f"entry {i} names block {e.block} of {len(self.blocks)}")

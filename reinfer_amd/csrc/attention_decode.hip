@@ -53,9 +53,11 @@ struct FdCut {
   int n;       // chunks
 };
 // gran: keys a workgroup takes a round (its waves x 32); a chunk is a whole number of rounds
-__device__ __forceinline__ FdCut fd_cut(int p, int lo, int chunk_shift, int max_chunks, int gran) {
+// keep16: the kept first keys below the window, in whole tiles (fd_kept): they are cut along with the window's
+// keys, standing right below its first tile.
+__device__ __forceinline__ FdCut fd_cut(int p, int lo, int keep16, int chunk_shift, int max_chunks, int gran) {
   FdCut c;
-  c.base = lo & ~15;
+  c.base = (lo & ~15) - keep16;
   const int span = p - c.base + 1;
   int want = (span + (1 << chunk_shift) - 1) >> chunk_shift;       // chunk_min = 1 << chunk_shift
   want = want < max_chunks ? want : max_chunks;
@@ -65,17 +67,28 @@ __device__ __forceinline__ FdCut fd_cut(int p, int lo, int chunk_shift, int max_
   return c;
 }
 
+// A window may keep the request's first `keep` keys (key < keep is seen whatever its distance). Their tiles that
+// lie below the window's first tile, this many keys:
+__device__ __forceinline__ int fd_kept(int keep, int lo) {
+  const int want = (keep + 15) & ~15, room = lo & ~15;
+  return want < room ? want : room;
+}
+
 // EXACT: the head size is DMAX itself, so every test against it is decided when the kernel is compiled
-// MOD: the scores are changed before the softmax (RaScoreMod: a tanh cap, a per-head distance term)
-template <int DMAX, bool EXACT, int FD_WAVES, bool MOD>
+// FLAGS & FD_MOD: the scores are changed before the softmax (RaScoreMod: a tanh cap, a per-head distance term)
+// FLAGS & FD_KEEP: a window that keeps the first keys. The walk is over one run of places: from the window's first
+// tile on a place is the key's own number, and the kept tiles take the places right below it.
+enum { FD_MOD = 1, FD_KEEP = 2 };
+template <int DMAX, bool EXACT, int FD_WAVES, int FLAGS>
 __global__ void __launch_bounds__(FD_WAVES * RA_WAVE, (DMAX <= 128 && FD_WAVES == 4) ? 3 : 1)
 flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
                     const bf16_t* __restrict__ kcache, const bf16_t* __restrict__ vcache,
                     const int* __restrict__ block_tables, int max_blocks,
                     const int* __restrict__ token_list, const int* __restrict__ seq_of_token,
                     const int* __restrict__ positions, int block_size, int Hkv, int G, int d_arg,
-                    float scale_log2, int window, int chunk_shift, int max_chunks, int n_tokens,
+                    float scale_log2, int window, int keep, int chunk_shift, int max_chunks, int n_tokens,
                     int t_base, float* __restrict__ part_o, float* __restrict__ part_ml, float scale, RaScoreMod mod) {
+  constexpr bool MOD = (FLAGS & FD_MOD) != 0, KEEP = (FLAGS & FD_KEEP) != 0;
   constexpr int FD_THREADS = FD_WAVES * RA_WAVE;
   const int d = EXACT ? DMAX : d_arg;
   constexpr int NDT = DMAX / 32;       // 32-wide d tiles of the score product
@@ -98,8 +111,13 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
     const int seq = seq_of_token ? seq_of_token[t] : t;
     const int p = positions[t];
     const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-    const FdCut cut = fd_cut(p, lo, chunk_shift, max_chunks, FD_WAVES * 32);
+    const int keep16 = KEEP ? fd_kept(keep, lo) : 0;
+    const FdCut cut = fd_cut(p, lo, keep16, chunk_shift, max_chunks, FD_WAVES * 32);
     const int n_chunks = cut.n;
+    // a place's key: itself, or for the kept tiles, which stand below the window's first, the distance from the walk's start
+    const int win_at = lo & ~15;
+    auto key_of = [&](int place) -> int { return (KEEP && place < win_at) ? place - (win_at - keep16) : place; };
+    auto seen = [&](int key) -> bool { return key <= p && (key >= lo || (KEEP && key < keep)); };
     if (ci >= n_chunks) continue;
     const int* table = block_tables + (size_t)seq * max_blocks;
 
@@ -130,7 +148,7 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
     // costs what the trip did.)
     auto block_of = [&](int kt_any) -> int {
       const int kt = __builtin_amdgcn_readfirstlane(kt_any);
-      return (kt <= p && kt + 15 >= lo && kt < k_end) ? table[kt / block_size] : 0;
+      return (kt <= p && (KEEP || kt + 15 >= lo) && kt < k_end) ? table[key_of(kt) / block_size] : 0;
     };
     int next_blk[2];
     next_blk[0] = block_of(k_begin + wave * 32);
@@ -139,7 +157,7 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
       const int blk_now[2] = {next_blk[0], next_blk[1]};
       next_blk[0] = block_of(k0 + FD_WAVES * 32);
       next_blk[1] = block_of(k0 + FD_WAVES * 32 + 16);
-      if (k0 + 31 < lo) continue;
+      if (!KEEP && k0 + 31 < lo) continue;
       // the two 16-key tiles of this step; a tile past the last key is not touched
       bool live[2], edge[2];
       const bf16_t* kb[2];
@@ -147,10 +165,10 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
 #pragma unroll
       for (int tt = 0; tt < 2; ++tt) {
         const int kt = k0 + tt * 16;
-        live[tt] = kt <= p && kt + 15 >= lo;
+        live[tt] = kt <= p && (KEEP || kt + 15 >= lo);        // with kept keys every tile of the walk holds a key that is seen
         edge[tt] = kt + 15 > p || kt < lo;
         const int blk = live[tt] ? blk_now[tt] : 0;
-        const size_t tile = ((size_t)blk * Hkv + kvh) * block_size * d + (size_t)((kt % block_size) >> 4) * 16 * d;
+        const size_t tile = ((size_t)blk * Hkv + kvh) * block_size * d + (size_t)((key_of(kt) % block_size) >> 4) * 16 * d;
         kb[tt] = kcache + tile + (g * 16 + r) * 8;        // chunk 4 dt + g of slot r
         vb[tt] = vcache + tile + (g * 16 + r) * 4;        // slots 4g..4g+3 of row 16 ot + r
       }
@@ -183,9 +201,9 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
       for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int key = k0 + tt * 16 + 4 * g + i;
+          const int key = key_of(k0 + tt * 16) + 4 * g + i;
           float v = -INFINITY;
-          if (key <= p && key >= lo) {
+          if (seen(key)) {
             if (MOD) v = ra_mod_score_fast(s[tt][i] * scale, mod.softcap, inv_cap, biased, r1h, r2h, p - key) * 1.4426950408889634f;
             else v = s[tt][i] * scale_log2;
           }
@@ -214,8 +232,8 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
         if (edge[tt]) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            const int key = k0 + tt * 16 + 4 * g + i;
-            if (!(key <= p && key >= lo)) {
+            const int key = key_of(k0 + tt * 16) + 4 * g + i;
+            if (!seen(key)) {
 #pragma unroll
               for (int ot = 0; ot < NOT; ++ot) vreg[tt][ot][i] = (bf16_t)0.f;
             }
@@ -292,7 +310,7 @@ template <int AHEAD>
 __global__ void __launch_bounds__(RA_WAVE)
 flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                           bf16_t* __restrict__ out, int out_stride, const int* __restrict__ token_list,
-                          const int* __restrict__ positions, int Hkv, int G, int d, int window, int chunk_shift,
+                          const int* __restrict__ positions, int Hkv, int G, int d, int window, int keep, int chunk_shift,
                           int max_chunks, int gran, int t_base) {
   const int head = blockIdx.x, li = blockIdx.y;
   const int lane = threadIdx.x;
@@ -317,7 +335,7 @@ flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restr
     }
     const int p = positions[t];
     const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-    const int n_chunks = fd_cut(p, lo, chunk_shift, max_chunks, gran).n;
+    const int n_chunks = fd_cut(p, lo, fd_kept(keep, lo), chunk_shift, max_chunks, gran).n;
     if (n_chunks == 1) return;                           // written by the first kernel
     const bool mine = lane < n_chunks;
     const float mc = mine ? mc_raw : -INFINITY, lc = mine ? lc_raw : 0.f;
@@ -345,7 +363,7 @@ flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restr
   }
   const int p = positions[t];
   const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-  const int n_chunks = fd_cut(p, lo, chunk_shift, max_chunks, gran).n;
+  const int n_chunks = fd_cut(p, lo, fd_kept(keep, lo), chunk_shift, max_chunks, gran).n;
   if (n_chunks == 1) return;                           // written by the first kernel
   float acc[4] = {0.f, 0.f, 0.f, 0.f};                 // d <= 256: up to 4 outputs a lane
   float mt = -INFINITY, lt = 0.f;
@@ -411,11 +429,14 @@ static size_t fd_lds_limit(void) {
 template <int DM, bool EX, int WV>
 static hipError_t fd_allow_lds(size_t lds) {
   if (lds <= 64 * 1024) return hipSuccess;
-  hipError_t e = hipFuncSetAttribute((const void*)flash_decode_kernel<DM, EX, WV, false>,
-                                     hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-  if (e != hipSuccess) return e;
-  return hipFuncSetAttribute((const void*)flash_decode_kernel<DM, EX, WV, true>, hipFuncAttributeMaxDynamicSharedMemorySize,
-                             (int)lds);
+  const void* forms[4] = {(const void*)flash_decode_kernel<DM, EX, WV, 0>, (const void*)flash_decode_kernel<DM, EX, WV, FD_MOD>,
+                          (const void*)flash_decode_kernel<DM, EX, WV, FD_KEEP>,
+                          (const void*)flash_decode_kernel<DM, EX, WV, FD_MOD | FD_KEEP>};
+  for (const void* f : forms) {
+    const hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return e;
+  }
+  return hipSuccess;
 }
 
 static int fd_resident_workgroups(int variant, int waves, size_t lds) {
@@ -431,8 +452,8 @@ static int fd_resident_workgroups(int variant, int waves, size_t lds) {
 #define RA_FD_OCC(DM)                                                                                                  \
   e = waves == 4 ? fd_allow_lds<DM, true, 4>(lds) : fd_allow_lds<DM, true, 12>(lds);                                   \
   if (e == hipSuccess)                                                                                                 \
-  e = waves == 4 ? hipOccupancyMaxActiveBlocksPerMultiprocessor(&per_cu, flash_decode_kernel<DM, true, 4, false>, 4 * RA_WAVE, lds) \
-                 : hipOccupancyMaxActiveBlocksPerMultiprocessor(&per_cu, flash_decode_kernel<DM, true, 12, false>, 12 * RA_WAVE, lds)
+  e = waves == 4 ? hipOccupancyMaxActiveBlocksPerMultiprocessor(&per_cu, flash_decode_kernel<DM, true, 4, 0>, 4 * RA_WAVE, lds) \
+                 : hipOccupancyMaxActiveBlocksPerMultiprocessor(&per_cu, flash_decode_kernel<DM, true, 12, 0>, 12 * RA_WAVE, lds)
   if (variant == 0) RA_FD_OCC(64);
   else if (variant == 1) RA_FD_OCC(128);
   else RA_FD_OCC(256);
@@ -472,7 +493,7 @@ extern "C" int ra_attention_decode(const void* q, int q_stride, void* out, int o
                                    int d, float scale, int window, int chunk, int max_chunks, int waves,
                                    float* part_o, float* part_ml, hipStream_t stream) {
   return ra_attention_decode_mod(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, token_list,
-                                 seq_of_token, positions, n_tokens, block_size, Hq, Hkv, d, scale, window, chunk,
+                                 seq_of_token, positions, n_tokens, block_size, Hq, Hkv, d, scale, window, 0, chunk,
                                  max_chunks, waves, part_o, part_ml, 0.f, nullptr, nullptr, stream);
 }
 
@@ -482,7 +503,7 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
                                        const void* kcache, const void* vcache, const int* block_tables,
                                        int max_blocks, const int* token_list, const int* seq_of_token,
                                        const int* positions, int n_tokens, int block_size, int Hq, int Hkv,
-                                       int d, float scale, int window, int chunk, int max_chunks, int waves,
+                                       int d, float scale, int window, int keep, int chunk, int max_chunks, int waves,
                                        float* part_o, float* part_ml, float softcap, const float* r1,
                                        const float* r2, hipStream_t stream) {
   RA_CHECK((r1 == nullptr) == (r2 == nullptr) && softcap >= 0.f,
@@ -493,7 +514,8 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
   RA_CHECK(ra_attention_decode_supports(Hq, Hkv, d, block_size),
            "attention_decode: unsupported sizes (%d query heads, %d KV heads, head size %d, block %d)", Hq,
            Hkv, d, block_size);
-  RA_CHECK(max_blocks > 0 && window >= 0, "attention_decode: bad cache geometry");
+  RA_CHECK(max_blocks > 0 && window >= 0 && keep >= 0, "attention_decode: bad cache geometry");
+  if (window == 0) keep = 0;                      // without a window every key is seen
   RA_CHECK(chunk >= 128 && (chunk & (chunk - 1)) == 0, "attention_decode: chunk %d is no power of two from 128", chunk);
   if (waves == 0) waves = 4;
   RA_CHECK(waves == 4 || waves == 12, "attention_decode: workgroups of %d waves (4 or 12)", waves);
@@ -517,13 +539,15 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
 #define RA_FD_ARGS                                                                                    \
   (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache, (const bf16_t*)vcache, \
       block_tables, max_blocks, token_list, seq_of_token, positions, block_size, Hkv, G, d, scale_log2, \
-      window, chunk_shift, max_chunks, n_tokens, 0, part_o, part_ml, scale, mod
+      window, keep, chunk_shift, max_chunks, n_tokens, 0, part_o, part_ml, scale, mod
 #define RA_FD_GO(DM, EX, WV)                                                                          \
   do {                                                                                                \
     if (fd_allow_lds<DM, EX, WV>(lds) != hipSuccess)                                                  \
       return ra_fail("attention_decode: the device does not give a workgroup %zu bytes of LDS", lds); \
-    if (changed) flash_decode_kernel<DM, EX, WV, true><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); \
-    else flash_decode_kernel<DM, EX, WV, false><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS);     \
+    if (changed && keep > 0) flash_decode_kernel<DM, EX, WV, FD_MOD | FD_KEEP><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); \
+    else if (changed) flash_decode_kernel<DM, EX, WV, FD_MOD><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); \
+    else if (keep > 0) flash_decode_kernel<DM, EX, WV, FD_KEEP><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); \
+    else flash_decode_kernel<DM, EX, WV, 0><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS);         \
   } while (0)
 #define RA_FD(DM)                                                                                     \
   do {                                                                                                \
@@ -547,7 +571,7 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
     dim3 mg(Hq, n_tokens);
 #define RA_FDM(AH)                                                                                          \
   flash_decode_merge_kernel<AH><<<mg, RA_WAVE, 0, stream>>>(part_o, part_ml, (bf16_t*)out, out_stride, token_list, \
-                                                           positions, Hkv, G, d, window, chunk_shift, max_chunks, waves * 32, 0)
+                                                           positions, Hkv, G, d, window, keep, chunk_shift, max_chunks, waves * 32, 0)
     if (max_chunks > FDM_AHEAD) RA_FDM(0);
     else if (d <= 64) RA_FDM(1);
     else if (d <= 128) RA_FDM(2);

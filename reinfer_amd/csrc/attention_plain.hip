@@ -5,7 +5,8 @@
 //
 //   s_t = scale * (q . K_t) for keys t in [lo, p] of the token's own request,
 //   lo = max(0, p - window + 1) if window > 0 else 0; softmax with the running
-//   maximum subtracted; o = sum_t P_t V_t.
+//   maximum subtracted; o = sum_t P_t V_t. With keep > 0 the first keep keys of the
+//   request are seen as well, however far the window has moved.
 //   Query head a reads KV head a / (Hq / Hkv).
 //   With a score change (RaScoreMod): s <- cap tanh(s / cap) where cap > 0, then
 //   s <- s - r1[a] ln(1 + r2[a] (p - t)) where the two per-head vectors are given.
@@ -22,7 +23,7 @@ __global__ void attention_plain_kernel(const TA* __restrict__ q, int q_stride, T
                                        const int* __restrict__ token_list,
                                        const int* __restrict__ seq_of_token,
                                        const int* __restrict__ positions, int block_size, int Hq,
-                                       int Hkv, int d, float scale, int window, RaScoreMod mod) {
+                                       int Hkv, int d, float scale, int window, int keep, RaScoreMod mod) {
   extern __shared__ float lds[];          // q vector [d], then probabilities [64]
   float* qs = lds;
   float* ps = lds + d;
@@ -44,10 +45,14 @@ __global__ void attention_plain_kernel(const TA* __restrict__ q, int q_stride, T
   for (int i = 0; i < 16; ++i) acc[i] = 0.f;
   float m = -INFINITY, l = 0.f;
 
-  for (int base = lo; base <= p; base += RA_WAVE) {
-    const int key = base + lane;
+  // the keys seen, in order: the kept first ones below the window, then the window
+  const int n_kept = keep < lo ? keep : lo;
+  const int n_seen = n_kept + p - lo + 1;
+  for (int base = 0; base < n_seen; base += RA_WAVE) {
+    const int at = base + lane;
+    const int key = at < n_kept ? at : lo + at - n_kept;
     float s = -INFINITY;
-    if (key <= p) {
+    if (at < n_seen) {
       const int blk = table[key / block_size];
       const TA* kr = kcache + ((size_t)blk * Hkv + kvh) * block_size * d;
       const int off = key % block_size;
@@ -58,14 +63,14 @@ __global__ void attention_plain_kernel(const TA* __restrict__ q, int q_stride, T
     }
     const float cmax = wave_max(s);
     const float m_new = fmaxf(m, cmax);
-    const float pr = (key <= p) ? expf(s - m_new) : 0.f;
+    const float pr = (at < n_seen) ? expf(s - m_new) : 0.f;
     const float corr = (m == -INFINITY) ? 0.f : expf(m - m_new);
     l = l * corr + wave_sum(pr);
     m = m_new;
     __syncthreads();                 // ps of the previous chunk is no longer read
     ps[lane] = pr;
     __syncthreads();
-    const int n_keys = (p - base + 1 < RA_WAVE) ? p - base + 1 : RA_WAVE;
+    const int n_keys = (n_seen - base < RA_WAVE) ? n_seen - base : RA_WAVE;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       if (r < n_acc) {
@@ -73,7 +78,8 @@ __global__ void attention_plain_kernel(const TA* __restrict__ q, int q_stride, T
         float sum = 0.f;
         if (i < d) {
           for (int kk = 0; kk < n_keys; ++kk) {
-            const int key2 = base + kk;
+            const int at2 = base + kk;
+            const int key2 = at2 < n_kept ? at2 : lo + at2 - n_kept;
             const int blk = table[key2 / block_size];
             const TA* vr = vcache + ((size_t)blk * Hkv + kvh) * block_size * d;
             sum += ps[kk] * to_f32(vr[cache_v_index(key2 % block_size, i, d)]);
@@ -101,14 +107,14 @@ extern "C" int ra_attention_plain(const void* q, int q_stride, void* out, int ou
                                   int d, float scale, int window, hipStream_t stream) {
   return ra_attention_plain_mod(q, q_stride, out, out_stride, kcache, vcache, act_dtype, block_tables, max_blocks,
                                 token_list, seq_of_token, positions, n_tokens, block_size, Hq, Hkv, d, scale, window,
-                                0.f, nullptr, nullptr, stream);
+                                0, 0.f, nullptr, nullptr, stream);
 }
 
 extern "C" int ra_attention_plain_mod(const void* q, int q_stride, void* out, int out_stride,
                                       const void* kcache, const void* vcache, int act_dtype,
                                       const int* block_tables, int max_blocks, const int* token_list,
                                       const int* seq_of_token, const int* positions, int n_tokens, int block_size,
-                                      int Hq, int Hkv, int d, float scale, int window, float softcap,
+                                      int Hq, int Hkv, int d, float scale, int window, int keep, float softcap,
                                       const float* r1, const float* r2, hipStream_t stream) {
   RA_CHECK((r1 == nullptr) == (r2 == nullptr) && softcap >= 0.f,
            "attention_plain: the distance term takes both per-head vectors, the cap is not negative");
@@ -119,19 +125,19 @@ extern "C" int ra_attention_plain_mod(const void* q, int q_stride, void* out, in
   RA_CHECK(block_size > 0 && block_size % 16 == 0 && d % 16 == 0 && max_blocks > 0,
            "attention_plain: the cache is tiled 16 x 16: block size %d and head size %d must be multiples of 16",
            block_size, d);
-  RA_CHECK(window >= 0, "attention_plain: negative window");
+  RA_CHECK(window >= 0 && keep >= 0, "attention_plain: negative window or number of kept keys");
   RA_CHECK(n_tokens <= 65535, "attention_plain: %d tokens in one launch (max 65535)", n_tokens);
   dim3 grid(Hq, n_tokens);
   const size_t lds = (size_t)(d + RA_WAVE) * sizeof(float);
   if (act_dtype == RA_F32)
     attention_plain_kernel<float><<<grid, RA_WAVE, lds, stream>>>(
         (const float*)q, q_stride, (float*)out, out_stride, (const float*)kcache, (const float*)vcache,
-        block_tables, max_blocks, token_list, seq_of_token, positions, block_size, Hq, Hkv, d, scale, window, mod);
+        block_tables, max_blocks, token_list, seq_of_token, positions, block_size, Hq, Hkv, d, scale, window, keep, mod);
   else if (act_dtype == RA_BF16)
     attention_plain_kernel<bf16_t><<<grid, RA_WAVE, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache,
         (const bf16_t*)vcache, block_tables, max_blocks, token_list, seq_of_token, positions, block_size,
-        Hq, Hkv, d, scale, window, mod);
+        Hq, Hkv, d, scale, window, keep, mod);
   else
     return ra_fail("attention_plain: unknown dtype tag %d", act_dtype);
   RA_LAUNCH_CHECK("attention_plain");

@@ -25,7 +25,7 @@
 // tile's exponentials.
 //
 // Causal: a query at position p sees keys <= p (and > p - window if a window is
-// set). The reference's prompt attention is a vendored library kernel that sees
+// set, but for the request's first `keep` keys, which a window may keep in sight). The reference's prompt attention is a vendored library kernel that sees
 // only the prompt itself, from position 0 (crates/cuda/src/fmha.rs:574-686;
 // crates/cuda/kernels/fmha_kernels.cu:96); this one is written here and reads
 // earlier context from the cache, so a prompt can be cut anywhere.
@@ -68,16 +68,20 @@ struct FpSplit {
 };
 
 // EXACT: the head size is DMAX itself, so every test against it is decided when the kernel is compiled
-// MOD: the scores are changed before the softmax (RaScoreMod: a tanh cap, a per-head distance term); the scaled
+// FLAGS & FP_MOD: the scores are changed before the softmax (RaScoreMod: a tanh cap, a per-head distance term); the scaled
 // and changed score then replaces the product in the registers, and scale_log2 is log2(e) alone
-template <int DMAX, int NC, bool EXACT, bool MOD>
+// FLAGS & FP_KEEP: a window that keeps the first `keep` keys; the rounds that hold them and lie below the window's
+// first round are walked before it.
+enum { FP_MOD = 1, FP_KEEP = 2 };
+template <int DMAX, int NC, bool EXACT, int FLAGS>
 __global__ void __launch_bounds__(FP_THREADS)
 flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
                      const bf16_t* __restrict__ kcache, const bf16_t* __restrict__ vcache,
                      const int* __restrict__ block_tables, int max_blocks,
                      const int* __restrict__ tile_info,      // per tile: seq, first token row, n queries, first position
                      int block_size, int Hq, int Hkv, int d_arg, int HG, float scale_log2, int window,
-                     FpSplit sp, float mod_scale, RaScoreMod mod) {
+                     int keep, FpSplit sp, float mod_scale, RaScoreMod mod) {
+  constexpr bool MOD = (FLAGS & FP_MOD) != 0, KEEP = (FLAGS & FP_KEEP) != 0;
   const int d = EXACT ? DMAX : d_arg;
   constexpr int NDT = DMAX / 32;       // 32-wide d tiles of the score product
   constexpr int NOT = DMAX / 16;       // 16-row d tiles of the output
@@ -147,7 +151,8 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
   // keys this tile of queries can see, and this wave's share of them
   const int last_pos = pos0 + nq - 1;
   const int first_key = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
-  int kt_begin = first_key / FP_KT * FP_KT;
+  const int win_round = first_key / FP_KT * FP_KT;       // the round that holds the window's first key
+  int kt_begin = win_round;
   int k_stop = last_pos;                      // the last key of this workgroup's rounds
   int slot = -1;
   if (sp.ranges) {
@@ -155,6 +160,20 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
     k_stop = min(k_stop, sp.ranges[tile * 3 + 1] - 1);
     slot = sp.ranges[tile * 3 + 2];
   }
+  // Kept first keys below the window's first round: rounds [kept_from, kept_from + kept) of this workgroup's share
+  // take the places right below kt_begin; from there on a place is the key's own number.
+  int kept = 0, kept_from = 0;
+  if (KEEP) {
+    int kept_end = min((keep + FP_KT - 1) / FP_KT * FP_KT, win_round);
+    if (sp.ranges) {
+      kept_from = sp.ranges[tile * 3 + 0];
+      kept_end = min(kept_end, sp.ranges[tile * 3 + 1]);
+    }
+    kept = max(kept_end - kept_from, 0);
+    if (k_stop < kt_begin) k_stop = kt_begin - 1;        // nothing of the window in this share: the kept rounds alone
+  }
+  const int place_begin = kt_begin - kept;
+  auto key_of = [&](int place) -> int { return (KEEP && place < kt_begin) ? place - place_begin + kept_from : place; };
   const int w_q0 = (wave * NC / HG) * 16;                       // first query of the wave
   const int w_qend = ((wave * NC + NC - 1) / HG + 1) * 16;      // one past its last
   const int w_first_pos = pos0 + w_q0;
@@ -183,7 +202,7 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
     for (int u = 0; u < NPRE; ++u) {
       const int tt = __builtin_amdgcn_readfirstlane(tile_of(u));
       const int kt = k0 + tt * 16;
-      const bool live = kt <= k_stop && kt + 15 >= first_key;           // wave-uniform
+      const bool live = kt <= k_stop && (kt + 15 >= first_key || (KEEP && kt < keep));           // wave-uniform
       const int ktl = live ? kt : safe_kt;
       const int blk = table[ktl >> bs_shift];
       const size_t tile_at = (((size_t)blk * Hkv + kvh) << bs_shift) * d + (size_t)((ktl & (block_size - 1)) >> 4) * 16 * d;
@@ -200,17 +219,17 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
       const int kt = k0 + tt * 16;
       const bf16x8_t zero = {0, 0, 0, 0, 0, 0, 0, 0};
       bf16x8_t kv = F.kpre[u], vv = F.vpre[u];
-      if (!(kt <= last_pos && kt + 15 >= first_key)) {
+      if (!(kt <= last_pos && (kt + 15 >= first_key || (KEEP && kt < keep)))) {
         kv = zero;
         vv = zero;
       } else if (kt + 15 > last_pos || kt < first_key) {
         // slots of the tile outside the visible range may hold anything (a freed block's bits): zero them
         const int kkey = kt + (w & 15);                      // K chunk w: 8 elements of slot w % 16
-        if (kkey > last_pos || kkey < first_key) kv = zero;
+        if (kkey > last_pos || (kkey < first_key && !(KEEP && kkey < keep))) kv = zero;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {                        // V chunk w: slots 4 ((w / 8) % 4) + e % 4
           const int vkey = kt + ((w >> 3) & 3) * 4 + (e & 3);
-          if (vkey > last_pos || vkey < first_key) vv[e] = (bf16_t)0.f;
+          if (vkey > last_pos || (vkey < first_key && !(KEEP && vkey < keep))) vv[e] = (bf16_t)0.f;
         }
       }
       if (w < 2 * d) {
@@ -239,7 +258,7 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
     const bf16_t* Vs = Vs2[buf];
     // a wave whose queries all lie before this round, or that has none, has nothing to add
     if (w_last_pos < w_first_pos || w_last_pos < k0) return;
-    if (window > 0 && k0 + FP_KT - 1 < w_first_pos - window + 1) return;
+    if (window > 0 && k0 + FP_KT - 1 < w_first_pos - window + 1 && !(KEEP && k0 < keep)) return;
 
     // two halves of 32 keys, each: scores, online softmax, values
 #pragma unroll
@@ -315,7 +334,7 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
       }
       // keys strictly inside every query's view need no mask
       const bool inner = kh + 31 <= w_first_pos && w_qend <= nq &&
-                         (window <= 0 || kh >= w_last_pos - window + 1);
+                         (window <= 0 || kh >= w_last_pos - window + 1 || (KEEP && kh + 31 < keep));
       if (!inner) {
 #pragma unroll
         for (int j = 0; j < NC; ++j) {
@@ -326,7 +345,7 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
               const int key = kh + ks * 16 + 4 * g + i;
-              if (!(q_live[j] && key <= q_pos && key >= q_lo)) s[ks][j][i] = -INFINITY;
+              if (!(q_live[j] && key <= q_pos && (key >= q_lo || (KEEP && key < keep)))) s[ks][j][i] = -INFINITY;
             }
         }
       }
@@ -410,20 +429,20 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
   // wave that stages buffer b for round i has passed the barrier of round i - 1, which every wave
   // reaches only after its reads of round i - 2, the last user of buffer b.
   Fetched F0, F1;
-  fetch(F0, kt_begin);
+  fetch(F0, key_of(place_begin));
   __builtin_amdgcn_sched_barrier(0);
-  fetch(F1, kt_begin + FP_KT);
+  fetch(F1, key_of(place_begin + FP_KT));
   __builtin_amdgcn_sched_barrier(0);
-  for (int k0 = kt_begin; k0 <= k_stop; k0 += 2 * FP_KT) {       // the bounds are the same in every thread
-    stage(F0, k0, 0);
+  for (int k0 = place_begin; k0 <= k_stop; k0 += 2 * FP_KT) {       // the bounds are the same in every thread
+    stage(F0, key_of(k0), 0);
     __syncthreads();
-    fetch(F0, k0 + 2 * FP_KT);
-    compute(k0, 0);
+    fetch(F0, key_of(k0 + 2 * FP_KT));
+    compute(key_of(k0), 0);
     if (k0 + FP_KT > k_stop) break;
-    stage(F1, k0 + FP_KT, 1);
+    stage(F1, key_of(k0 + FP_KT), 1);
     __syncthreads();
-    fetch(F1, k0 + 3 * FP_KT);
-    compute(k0 + FP_KT, 1);
+    fetch(F1, key_of(k0 + 3 * FP_KT));
+    compute(key_of(k0 + FP_KT), 1);
   }
 #pragma unroll
   for (int j = 0; j < NC; ++j) {
@@ -580,7 +599,7 @@ extern "C" long ra_attention_prefill_part_floats(int Hq, int Hkv, int d, int n_s
 static int fp_launch(const void* q, int q_stride, void* out, int out_stride,
                      const void* kcache, const void* vcache, const int* block_tables,
                      int max_blocks, const int* tile_info, int n_tiles, int block_size,
-                     int Hq, int Hkv, int d, float scale, int window, const FpSplit& sp, const int* merge_info,
+                     int Hq, int Hkv, int d, float scale, int window, int keep, const FpSplit& sp, const int* merge_info,
                      int n_merge, const RaScoreMod& mod, hipStream_t stream) {
   RA_CHECK((mod.r1 == nullptr) == (mod.r2 == nullptr) && mod.softcap >= 0.f,
            "attention_prefill: the distance term takes both per-head vectors, the cap is not negative");
@@ -589,7 +608,8 @@ static int fp_launch(const void* q, int q_stride, void* out, int out_stride,
   RA_CHECK(ra_attention_prefill_supports(Hq, Hkv, d, block_size),
            "attention_prefill: unsupported sizes (%d query heads, %d KV heads, head size %d, block %d)", Hq,
            Hkv, d, block_size);
-  RA_CHECK(max_blocks > 0 && window >= 0, "attention_prefill: bad cache geometry");
+  RA_CHECK(max_blocks > 0 && window >= 0 && keep >= 0, "attention_prefill: bad cache geometry");
+  if (window == 0) keep = 0;                      // without a window every key is seen
   RA_CHECK(q_stride % 8 == 0 && out_stride % 4 == 0 && ((uintptr_t)q % 16) == 0 && ((uintptr_t)out % 8) == 0 &&
                ((uintptr_t)kcache % 16) == 0 && ((uintptr_t)vcache % 16) == 0,
            "attention_prefill: operands must be 16-byte aligned");
@@ -602,11 +622,13 @@ static int fp_launch(const void* q, int q_stride, void* out, int out_stride,
   const float scale_log2 = (changed ? 1.f : scale) * 1.4426950408889634f;
 #define RA_FP_ARGS                                                                                    \
   (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache, (const bf16_t*)vcache, \
-      block_tables, max_blocks, tile_info, block_size, Hq, Hkv, d, sh.hg, scale_log2, window, sp, scale, mod
+      block_tables, max_blocks, tile_info, block_size, Hq, Hkv, d, sh.hg, scale_log2, window, keep, sp, scale, mod
 #define RA_FP_GO(DM, NCC, EX)                                                                         \
   do {                                                                                                \
-    if (changed) flash_prefill_kernel<DM, NCC, EX, true><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
-    else flash_prefill_kernel<DM, NCC, EX, false><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS);       \
+    if (changed && keep > 0) flash_prefill_kernel<DM, NCC, EX, FP_MOD | FP_KEEP><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
+    else if (changed) flash_prefill_kernel<DM, NCC, EX, FP_MOD><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
+    else if (keep > 0) flash_prefill_kernel<DM, NCC, EX, FP_KEEP><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
+    else flash_prefill_kernel<DM, NCC, EX, 0><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS);           \
   } while (0)
 #define RA_FP(DM, NCC)                                                                                \
   do {                                                                                                \
@@ -640,7 +662,7 @@ extern "C" int ra_attention_prefill(const void* q, int q_stride, void* out, int 
                                     int max_blocks, const int* tile_info, int n_tiles, int block_size,
                                     int Hq, int Hkv, int d, float scale, int window, hipStream_t stream) {
   return ra_attention_prefill_mod(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, tile_info,
-                                  n_tiles, block_size, Hq, Hkv, d, scale, window, 0.f, nullptr, nullptr, stream);
+                                  n_tiles, block_size, Hq, Hkv, d, scale, window, 0, 0.f, nullptr, nullptr, stream);
 }
 
 // The same with the scores changed before the softmax: softcap > 0 caps them by a tanh, r1 / r2 (one float a query
@@ -648,12 +670,12 @@ extern "C" int ra_attention_prefill(const void* q, int q_stride, void* out, int 
 extern "C" int ra_attention_prefill_mod(const void* q, int q_stride, void* out, int out_stride,
                                         const void* kcache, const void* vcache, const int* block_tables,
                                         int max_blocks, const int* tile_info, int n_tiles, int block_size,
-                                        int Hq, int Hkv, int d, float scale, int window, float softcap,
+                                        int Hq, int Hkv, int d, float scale, int window, int keep, float softcap,
                                         const float* r1, const float* r2, hipStream_t stream) {
   const FpSplit none = {};
   const RaScoreMod mod = {softcap, r1, r2};
   return fp_launch(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, tile_info, n_tiles,
-                   block_size, Hq, Hkv, d, scale, window, none, nullptr, 0, mod, stream);
+                   block_size, Hq, Hkv, d, scale, window, keep, none, nullptr, 0, mod, stream);
 }
 
 // The same with query tiles cut by keys: `ranges` holds three ints a listed tile (first key and one past the
@@ -668,14 +690,14 @@ extern "C" int ra_attention_prefill_split(const void* q, int q_stride, void* out
                                           hipStream_t stream) {
   return ra_attention_prefill_split_mod(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks,
                                         tile_info, n_tiles, ranges, merge_info, n_merge, part_o, part_ml, block_size,
-                                        Hq, Hkv, d, scale, window, 0.f, nullptr, nullptr, stream);
+                                        Hq, Hkv, d, scale, window, 0, 0.f, nullptr, nullptr, stream);
 }
 
 extern "C" int ra_attention_prefill_split_mod(const void* q, int q_stride, void* out, int out_stride,
                                               const void* kcache, const void* vcache, const int* block_tables,
                                               int max_blocks, const int* tile_info, int n_tiles, const int* ranges,
                                               const int* merge_info, int n_merge, float* part_o, float* part_ml,
-                                              int block_size, int Hq, int Hkv, int d, float scale, int window,
+                                              int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
                                               float softcap, const float* r1, const float* r2, hipStream_t stream) {
   const RaScoreMod mod = {softcap, r1, r2};
   RA_CHECK(ranges && merge_info && n_merge > 0 && part_o && part_ml,
@@ -686,5 +708,5 @@ extern "C" int ra_attention_prefill_split_mod(const void* q, int q_stride, void*
   sp.part_o = part_o;
   sp.part_ml = part_ml;
   return fp_launch(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, tile_info, n_tiles,
-                   block_size, Hq, Hkv, d, scale, window, sp, merge_info, n_merge, mod, stream);
+                   block_size, Hq, Hkv, d, scale, window, keep, sp, merge_info, n_merge, mod, stream);
 }

@@ -315,7 +315,8 @@ extern "C" int ra_add_group_rmsnorm(float* resid, const void* delta, const void*
 // Fused per-head RMSNorm of q and k, rotation, and cache write.
 // qkv: [T, (Hq + 2 Hkv) * d]; q heads are normalised + rotated in place, k heads
 // are normalised + rotated and stored at the token's cache slot, v heads are
-// copied there. One wavefront per (token, head).
+// copied there. One wavefront per (token, head). Where a layer's values are its keys as projected (v_back = Hkv,
+// else 0) a row holds q and k alone, (Hq + Hkv) * d, and a v head reads its k head's row before the norm.
 //   head norm: u * rsqrt(mean(u^2) + eps) * g, one g[d] for all heads, before the
 //     rotation (crates/cuda/kernels/dense_kernels.cu:92-123; engine.rs:4122-4147)
 //   rotation: pairs (j, j + R/2) [style 0, half split] or (2j, 2j+1) [style 1],
@@ -347,7 +348,7 @@ __global__ void qk_norm_rope_cache_kernel(TA* __restrict__ qkv, const TW* __rest
                                           const float* __restrict__ inv_freq, int rotary_dim,
                                           int rope_style, const int* __restrict__ slots,
                                           TA* __restrict__ kcache, TA* __restrict__ vcache,
-                                          int block_size, int Hq, int Hkv, int d, QkSums sm) {
+                                          int block_size, int Hq, int Hkv, int d, int v_back, QkSums sm) {
   __shared__ float buf[QK_WAVES][QK_MAX_D];
   const int lane = threadIdx.x & (RA_WAVE - 1);
   const int wave = threadIdx.x / RA_WAVE;
@@ -355,9 +356,11 @@ __global__ void qk_norm_rope_cache_kernel(TA* __restrict__ qkv, const TW* __rest
   const int head = blockIdx.x * QK_WAVES + wave;
   const int n_heads = Hq + 2 * Hkv;
   const bool live = head < n_heads;
-  TA* u = qkv + ((size_t)t * n_heads + (live ? head : 0)) * d;
   const bool is_q = head < Hq;
   const bool is_k = !is_q && head < Hq + Hkv;
+  const int row_heads = n_heads - v_back;
+  const int src_head = (is_q || is_k) ? head : head - v_back;      // the head of the row that holds this one's elements
+  TA* u = qkv + ((size_t)t * row_heads + (live ? src_head : 0)) * d;
   const int kvh = is_q ? 0 : (is_k ? head - Hq : head - Hq - Hkv);
   const int slot = slots[t];
   TA* slab = nullptr;           // the (block, kv head) slab a k or v head goes to
@@ -378,7 +381,7 @@ __global__ void qk_norm_rope_cache_kernel(TA* __restrict__ qkv, const TW* __rest
         tsum = wave_sum(tsum);
         row = rsqrtf(tsum * sm.in_inv_width + sm.in_eps);
       }
-      const float* src = sm.parts + ((size_t)t * n_heads + head) * d;
+      const float* src = sm.parts + ((size_t)t * row_heads + src_head) * d;
       for (int i = lane; i < d; i += RA_WAVE) {
         float v = 0.f;                         // range order; six ranges' values asked for in one trip
         constexpr int U = 6;
@@ -462,7 +465,7 @@ __global__ void __launch_bounds__(QK_WAVES * RA_WAVE)
 qk_norm_rope_cache_head_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w, const TW* __restrict__ k_w,
                                float eps, const int* __restrict__ positions, const float* __restrict__ inv_freq,
                                const int* __restrict__ slots, TA* __restrict__ kcache, TA* __restrict__ vcache,
-                               int block_size, int Hq, int Hkv) {
+                               int block_size, int Hq, int Hkv, int v_back) {
   constexpr int d = 64 * EPL;
   constexpr int NF = EPL >= 2 ? EPL / 2 : 1;
   const int lane = threadIdx.x & (RA_WAVE - 1);
@@ -471,9 +474,9 @@ qk_norm_rope_cache_head_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w,
   const int head = blockIdx.x * QK_WAVES + wave;
   const int n_heads = Hq + 2 * Hkv;
   if (head >= n_heads) return;
-  TA* u = qkv + ((size_t)t * n_heads + head) * d;
   const bool is_q = head < Hq;
   const bool is_k = !is_q && head < Hq + Hkv;
+  TA* u = qkv + ((size_t)t * (n_heads - v_back) + ((is_q || is_k) ? head : head - v_back)) * d;
   const TW* w = is_q ? q_w : k_w;              // a v head reads k's weights and drops them
   // ---- every load, then the first use
   const int slot = slots[t];
@@ -595,7 +598,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
                                 float eps, const int* __restrict__ positions,
                                 const float* __restrict__ inv_freq, const int* __restrict__ slots,
                                 TA* __restrict__ kcache, TA* __restrict__ vcache, int block_size, int Hq,
-                                int Hkv, int d, int T, int share) {
+                                int Hkv, int d, int v_back, int T, int share) {
   constexpr int E = Row16<TA>::E;
   constexpr int ROWS = 256 / LPH;              // head rows a pass of the workgroup
   extern __shared__ __attribute__((aligned(16))) unsigned char qk_lds[];
@@ -609,7 +612,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
   const int w_xcd = blockIdx.x % RA_XCDS, w_k = blockIdx.x / RA_XCDS;
   const int t = ((w_k / 16) * RA_XCDS + w_xcd) * 16 + w_k % 16;
   if (t >= T) return;
-  const int n_heads = Hq + 2 * Hkv;
+  const int n_heads = Hq + 2 * Hkv - v_back;   // heads of a row
   const int sub = threadIdx.x / LPH, ln = threadIdx.x % LPH;
   const int j0 = ln * E;                       // pairs j0..j0+E-1
   const int slot = slots[t];
@@ -686,7 +689,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
     for (int r = sub; r < 2 * Hkv; r += ROWS) {
       const bool is_k = r < Hkv;
       const int kvh = is_k ? r : r - Hkv;
-      const TA* u = qkv + ((size_t)t * n_heads + Hq + r) * d;
+      const TA* u = qkv + ((size_t)t * n_heads + Hq + (is_k ? r : r - v_back)) * d;
       TA* slab = (is_k ? kcache : vcache) + (blk * Hkv + kvh) * (size_t)block_size * d;
       if (is_k) {                              // the elements of one 8-chunk are contiguous in the K tile
         float ra[E], rc[E];
@@ -718,7 +721,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
     const int m = r >> 3, tok = r & 3;
     const bool is_k = (r & 4) == 0;
     const int kvh = me + 4 * m;
-    const TA* u = qkv + ((size_t)(t0 + tok) * n_heads + Hq + (is_k ? 0 : Hkv) + kvh) * d;
+    const TA* u = qkv + ((size_t)(t0 + tok) * n_heads + Hq + (is_k ? 0 : Hkv - v_back) + kvh) * d;
     if (is_k) {
       float ra[E], rc[E];
       turn(u, k_w, tok, ra, rc);
@@ -769,7 +772,8 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
                                    int weight_dtype, float eps, const int* positions,
                                    const float* inv_freq, int rotary_dim, int rope_style,
                                    const int* slots, void* kcache, void* vcache, int block_size,
-                                   int n_tokens, int Hq, int Hkv, int d, const QkSums& sm, hipStream_t stream) {
+                                   int n_tokens, int Hq, int Hkv, int d, int values_are_keys, const QkSums& sm, hipStream_t stream) {
+  const int v_back = values_are_keys ? Hkv : 0;
   RA_CHECK(n_tokens > 0, "qk_norm_rope_cache: no tokens");
   RA_CHECK(Hq > 0 && Hkv > 0 && d > 0, "qk_norm_rope_cache: bad head sizes (%d, %d, %d)", Hq, Hkv, d);
   RA_CHECK(d <= QK_MAX_D, "qk_norm_rope_cache: head size %d above the supported %d", d, QK_MAX_D);
@@ -794,7 +798,7 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
       <<<(n_tokens + 16 * RA_XCDS - 1) / (16 * RA_XCDS) * (16 * RA_XCDS), 256,                            \
          qk_token_lds(Hkv, d, sizeof(TA), share), stream>>>(                                              \
       (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, slots, (TA*)kcache,  \
-      (TA*)vcache, block_size, Hq, Hkv, d, n_tokens, share ? 1 : 0)
+      (TA*)vcache, block_size, Hq, Hkv, d, v_back, n_tokens, share ? 1 : 0)
   /* lanes a head: 16 bytes of either half a lane (SH: 0 for 4-byte elements, 1 for 2-byte ones) */
 #define RA_TOK(TA, TW, SH)                           \
   do {                                               \
@@ -820,11 +824,11 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
     if (q_weight)                                                                                         \
       qk_norm_rope_cache_head_kernel<TA, TW, EPL, true><<<grid, QK_WAVES * RA_WAVE, 0, stream>>>(         \
           (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, slots, (TA*)kcache, \
-          (TA*)vcache, block_size, Hq, Hkv);                                                              \
+          (TA*)vcache, block_size, Hq, Hkv, v_back);                                                              \
     else                                                                                                  \
       qk_norm_rope_cache_head_kernel<TA, TW, EPL, false><<<grid, QK_WAVES * RA_WAVE, 0, stream>>>(        \
           (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, slots, (TA*)kcache, \
-          (TA*)vcache, block_size, Hq, Hkv);                                                              \
+          (TA*)vcache, block_size, Hq, Hkv, v_back);                                                              \
   } while (0)
 #define RA_HEAD(TA, TW)                      \
   do {                                       \
@@ -844,7 +848,7 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
 #define RA_GO(TA, TW)                                                                              \
   qk_norm_rope_cache_kernel<TA, TW><<<grid, QK_WAVES * RA_WAVE, 0, stream>>>(                      \
       (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, rotary_dim,   \
-      rope_style, slots, (TA*)kcache, (TA*)vcache, block_size, Hq, Hkv, d, sm)
+      rope_style, slots, (TA*)kcache, (TA*)vcache, block_size, Hq, Hkv, d, v_back, sm)
   if (act_dtype == RA_F32 && weight_dtype == RA_F32) RA_GO(float, float);
   else if (act_dtype == RA_BF16 && weight_dtype == RA_BF16) RA_GO(bf16_t, bf16_t);
   else if (act_dtype == RA_BF16 && weight_dtype == RA_F32) RA_GO(bf16_t, float);
@@ -858,12 +862,12 @@ extern "C" int ra_qk_norm_rope_cache(void* qkv, int act_dtype, const void* q_wei
                                      int weight_dtype, float eps, const int* positions,
                                      const float* inv_freq, int rotary_dim, int rope_style,
                                      const int* slots, void* kcache, void* vcache, int block_size,
-                                     int n_tokens, int Hq, int Hkv, int d, hipStream_t stream) {
+                                     int n_tokens, int Hq, int Hkv, int d, int values_are_keys, hipStream_t stream) {
   RA_CHECK(qkv != nullptr, "qk_norm_rope_cache: no q/k/v rows");
   const QkSums none = {};
   return qk_norm_rope_cache_impl(qkv, act_dtype, q_weight, k_weight, weight_dtype, eps, positions, inv_freq,
                                  rotary_dim, rope_style, slots, kcache, vcache, block_size, n_tokens, Hq, Hkv, d,
-                                 none, stream);
+                                 values_are_keys, none, stream);
 }
 
 // The same from the float partial results of a product cut into K ranges ([n_ranges][n_tokens][width],
@@ -876,7 +880,7 @@ extern "C" int ra_qk_norm_rope_cache_sums(const float* parts, int n_ranges, cons
                                           float eps, const int* positions, const float* inv_freq,
                                           int rotary_dim, int rope_style, const int* slots, void* kcache,
                                           void* vcache, int block_size, int n_tokens, int Hq, int Hkv, int d,
-                                          hipStream_t stream) {
+                                          int values_are_keys, hipStream_t stream) {
   RA_CHECK(parts && n_ranges >= 1 && q_out, "qk_norm_rope_cache_sums: partial results and a place for q are needed");
   RA_CHECK(q_stride >= Hq * d, "qk_norm_rope_cache_sums: q rows of %d elements do not hold %d heads of %d", q_stride, Hq, d);
   RA_CHECK(in_ss == nullptr || (in_parts > 0 && in_width > 0 && in_eps >= 0.f),
@@ -884,7 +888,7 @@ extern "C" int ra_qk_norm_rope_cache_sums(const float* parts, int n_ranges, cons
   QkSums sm = {};
   sm.parts = parts;
   sm.n_ranges = n_ranges;
-  sm.range_stride = (size_t)n_tokens * (size_t)(Hq + 2 * Hkv) * (size_t)d;
+  sm.range_stride = (size_t)n_tokens * (size_t)(Hq + (values_are_keys ? 1 : 2) * Hkv) * (size_t)d;
   sm.in_ss = in_ss;
   sm.in_parts = in_parts;
   sm.in_eps = in_eps;
@@ -893,7 +897,7 @@ extern "C" int ra_qk_norm_rope_cache_sums(const float* parts, int n_ranges, cons
   sm.q_stride = q_stride;
   return qk_norm_rope_cache_impl(nullptr, act_dtype, q_weight, k_weight, weight_dtype, eps, positions, inv_freq,
                                  rotary_dim, rope_style, slots, kcache, vcache, block_size, n_tokens, Hq, Hkv, d,
-                                 sm, stream);
+                                 values_are_keys, sm, stream);
 }
 
 // ---------------------------------------------------------------------------

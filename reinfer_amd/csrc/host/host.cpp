@@ -7,10 +7,10 @@
 // same needs form a group (all earlier keys, or a window of them); every group
 // has a pool of its own and every request one block table per group. Blocks are
 // taken lazily, when a step's tokens need them, given back when the request ends
-// or, in a window group, when the window has passed them, and used again, last
-// freed first (the reference's PagePool is LIFO the same way,
-// crates/memory/src/pool.rs:61-155). Beside the pools: slots for per-request
-// state of fixed size.
+// or, in a window group, when the window has passed them (the first tokens that a
+// group's window keeps in sight stay), and used again, last freed first (the
+// reference's PagePool is LIFO the same way, crates/memory/src/pool.rs:61-155).
+// Beside the pools: slots for per-request state of fixed size.
 //
 // Scheduler: each call of schedule() decides one step: every decoding request
 // takes one token first; what is left of the token budget goes to prompt
@@ -147,7 +147,7 @@ struct RequestCache {
   int slot = 0;
   int num_tokens = 0;                          // tokens whose keys are stored
   std::vector<std::vector<int>> tables;        // per group; -1 = given back
-  std::vector<int> first_live;                 // per group: first block still held
+  std::vector<int> first_live;                 // per group: first block still held (kept first blocks aside)
   bool fresh = true;                           // no step has run for it yet
   uint64_t serial = 0;                         // distinguishes a request from an earlier one of the same id
 };
@@ -162,6 +162,7 @@ struct KeyEq {
 struct CacheManager {
   py::list groups;                             // the CacheGroupSpec records, as given
   std::vector<int> windows;
+  std::vector<int> keeps;                      // per group: first tokens that a window keeps in sight (0: none)
   int block_size;
   std::vector<BlockPool> pools;
   SlotPool slots;
@@ -172,7 +173,10 @@ struct CacheManager {
       : groups(groups_), block_size(block_size_), slots(max_seqs) {
     if (block_size <= 0) throw py::value_error("block_size must be positive");
     if (num_blocks.size() != (size_t)py::len(groups)) throw py::value_error("one block count per cache group");
-    for (auto g : groups) windows.push_back(g.attr("window").cast<int>());
+    for (auto g : groups) {
+      windows.push_back(g.attr("window").cast<int>());
+      keeps.push_back(py::hasattr(g, "keep") ? g.attr("keep").cast<int>() : 0);
+    }
     for (int n : num_blocks) pools.emplace_back(n);
   }
   int n_groups() const { return (int)windows.size(); }
@@ -215,14 +219,16 @@ struct CacheManager {
     const int lo = first_query_pos - w + 1;
     return std::max(0, lo) / block_size;
   }
+  // Blocks that hold the first tokens which group g's window keeps in sight: held as long as the request lives.
+  int kept_blocks(int g) const { return keeps[g] > 0 ? (keeps[g] + block_size - 1) / block_size : 0; }
   // Blocks each group must still take so that tokens [stored, new_total) fit.
   void blocks_needed_into(const RequestCache& rc, int new_total, int* need) const {
     const int want = (new_total + block_size - 1) / block_size;
     for (int g = 0; g < n_groups(); ++g) {
       const int have = (int)rc.tables[g].size();
-      // blocks wholly below the window of the first new query are never taken
+      // blocks wholly below the window of the first new query are never taken, but for the kept first ones
       const int first = std::max(have, first_needed_block(g, rc.num_tokens));
-      need[g] = std::max(0, want - first);
+      need[g] = std::max(0, want - first) + std::max(0, std::min({kept_blocks(g), want, first}) - have);
     }
   }
   std::vector<int> blocks_needed(const py::object& rid, int new_total) const {
@@ -252,7 +258,7 @@ struct CacheManager {
       auto& table = rc.tables[g];
       const int first = first_needed_block(g, rc.num_tokens);
       while ((int)table.size() < want) {
-        if ((int)table.size() < first) {
+        if ((int)table.size() < first && (int)table.size() >= kept_blocks(g)) {
           table.push_back(-1);                 // below the window from the start: never held
           rc.first_live[g] = (int)table.size();
         } else {
@@ -271,7 +277,7 @@ struct CacheManager {
       const int first = first_needed_block(g, new_total);       // the next query sits at new_total
       auto& table = rc.tables[g];
       const int end = std::min(first, (int)table.size());
-      for (int b = rc.first_live[g]; b < end; ++b)
+      for (int b = std::max(rc.first_live[g], kept_blocks(g)); b < end; ++b)
         if (table[b] >= 0) {
           pools[g].give_back(table[b]);
           table[b] = -1;

@@ -11,28 +11,9 @@
 // that loading and storing it are whole lines; nothing else reads it.
 #include "common.h"
 #include "reinfer_hip.h"
+#include "scan_geom.h"
 
 namespace {
-
-struct ScanGeom {
-  int R, NPL, CPW, waves;      // lanes a column, elements a lane, columns a wave, waves a head
-  int wave_floats;             // floats of state a wave
-};
-
-// kind 0: matrix memory (S, the normaliser n once a wave, the running maximum m); kind 1: delta rule (S);
-// kind 2: wkv (S); kind 3: a memory that fades by a constant a head (S)
-bool scan_geom(int kind, int dk, int dv, ScanGeom* g) {
-  if (dk <= 0 || dv <= 0 || dk > 512) return false;
-  // at most 8 elements a lane: the per-token chain of multiply-adds stays short, and a head has enough waves to
-  // spread over the chip when one request's prompt is all there is
-  g->R = dk <= 32 ? 8 : dk <= 128 ? 16 : dk <= 256 ? 32 : 64;
-  const int per = (dk + g->R - 1) / g->R;
-  g->NPL = per <= 2 ? 2 : per <= 4 ? 4 : 8;
-  g->CPW = RA_WAVE / g->R;
-  g->waves = (dv + g->CPW - 1) / g->CPW;
-  g->wave_floats = g->NPL * RA_WAVE + (kind == 0 ? g->NPL * g->R + 4 : 0);
-  return true;
-}
 
 // Sum over runs of R neighbouring lanes, every lane of a run getting the sum. Inside a row of 16 lanes the
 // exchanges are DPP operands of the adds (pairs, quads, the mirrored half row and row); only beyond 16 lanes does
@@ -52,9 +33,6 @@ __device__ __forceinline__ float group_sum(float v) {
   return v;
 }
 
-__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
-__device__ __forceinline__ float logsigmoid_f(float x) { return -softplus_f(-x); }
-
 // ---------------------------------------------------------------------------
 // The scan of either mixer. A workgroup (up to 4 waves: 32 or 8 columns of one head of one request) walks the
 // request's tokens in chunks: the chunk's k and q rows of the head (as floats, q scaled), the v entries of the
@@ -72,13 +50,17 @@ __device__ __forceinline__ float logsigmoid_f(float x) { return -softplus_f(-x);
 // u = beta (v - g a), o = g b + u kq, S <- g S + k u.
 // A memory that fades by a constant (DECAY): no gates; q, k and v pass silu as they are staged (float);
 //   S <- head_decay[h] S + k v^T;  o = S^T q   (the read-out sees the token's own write)
+// Retention (RETENTION): the same without silu; the first rot_dims elements of q and k turn by their position as they
+// are staged (pairs (i, i + rot_dims / 2), float), k times k_scale.
+// Gated linear attention (GLA): a decay a key channel and token, alpha = sigmoid(w + w0)^inv_tau, formed in float as
+// it is staged;  S <- diag(alpha) S + k v^T;  o = S^T q
 // ---------------------------------------------------------------------------
 #define SCAN_KQ_REGS 8         // k (and q) values a thread fetches for a chunk
 #define SCAN_V_REGS 2
 #define SCAN_CHUNK_MAX 16
 #define SCAN_LDS_FLOATS 6144   // of one of the two buffers
 
-enum { SCAN_DELTA = 0, SCAN_MEMORY = 1, SCAN_WKV = 2, SCAN_DECAY = 3 };
+enum { SCAN_DELTA = 0, SCAN_MEMORY = 1, SCAN_WKV = 2, SCAN_DECAY = 3, SCAN_RETENTION = 4, SCAN_GLA = 5 };
 
 struct ScanArgs {
   const void* q; const void* k; const void* v;     // column 0 of each in row 0; rows ld elements apart
@@ -92,17 +74,21 @@ struct ScanArgs {
   float* out;
   // wkv: the decays' pre-activations, float [T, H dk] with rows ldw apart, their bias w0 [H dk] and the bonus u [H dk]
   const float* w; int ldw; const float* w0; const float* u;
-  const float* head_decay;                           // the fading memory: one factor a head
+  const float* head_decay;                           // the fading memory, retention: one factor a head
+  float k_scale, inv_tau;                            // retention; gated linear attention
+  const int* positions; const float* inv_freq; int rot_dims;      // retention: the turn of q and k
 };
 
 template <typename TA, int R, int NPL, int MODE>
 __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
   constexpr bool MEMORY = MODE == SCAN_MEMORY, WKV = MODE == SCAN_WKV, DECAY = MODE == SCAN_DECAY;
+  constexpr bool RET = MODE == SCAN_RETENTION, GLA = MODE == SCAN_GLA;
+  constexpr bool CHANNEL = WKV || GLA;               // a decay a key channel and token, staged beside k and q
   constexpr int CPW = RA_WAVE / R;
   constexpr int PITCH = NPL + 4;                     // floats of a lane's run of k (or q) in LDS, padded
-  constexpr int NG = MEMORY ? 3 : (WKV || DECAY) ? 0 : 2;       // gate values a token
+  constexpr int NG = MEMORY ? 3 : (MODE != SCAN_DELTA) ? 0 : 2;       // gate values a token
   constexpr int NGD = NG ? NG : 1;
-  constexpr int NV = WKV ? 3 : 2;                    // vectors over the key size a token: k, q and, for wkv, the decay
+  constexpr int NV = CHANNEL ? 3 : 2;                // vectors over the key size a token: k, q and, a channel each, the decay
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int seq = blockIdx.x, head = blockIdx.y;
   const int tid = threadIdx.x, nthreads = blockDim.x;
@@ -132,10 +118,10 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
   const TA* kg = (const TA*)p.k + (size_t)qh * dk;
   const TA* vg = (const TA*)p.v + (size_t)head * dv + (size_t)blockIdx.z * cols;
   const int v_left = dv - blockIdx.z * cols;         // columns of this workgroup that exist
-  float fk[SCAN_KQ_REGS], fq[SCAN_KQ_REGS], fw[WKV ? SCAN_KQ_REGS : 1], fv[SCAN_V_REGS], fg = 0.f;
-  const float* wg = WKV ? p.w + (size_t)head * dk : nullptr;
-  const float* w0 = WKV ? p.w0 + (size_t)head * dk : nullptr;
-  int kq_w[WKV ? SCAN_KQ_REGS : 1];                  // the decay's place: rows of its own pitch, the bias by element
+  float fk[SCAN_KQ_REGS], fq[SCAN_KQ_REGS], fw[CHANNEL ? SCAN_KQ_REGS : 1], fv[SCAN_V_REGS], fg = 0.f;
+  const float* wg = CHANNEL ? p.w + (size_t)head * dk : nullptr;
+  const float* w0 = CHANNEL ? p.w0 + (size_t)head * dk : nullptr;
+  int kq_w[(CHANNEL || RET) ? SCAN_KQ_REGS : 1];     // the decay's place: rows of its own pitch, the bias by element
   // what this thread fetches for a chunk is the same for every chunk: token (of the chunk), offset behind the
   // chunk's first row, and place in LDS are worked out once
   int kq_t[SCAN_KQ_REGS], kq_g[SCAN_KQ_REGS], kq_l[SCAN_KQ_REGS];
@@ -148,7 +134,7 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
     kq_e[j] = e < dk;
     kq_g[j] = t * p.ld + e;
     kq_l[j] = t * NV * R * PITCH + (e / NPL) * PITCH + (e % NPL);
-    if (WKV) kq_w[j] = e;
+    if (CHANNEL || RET) kq_w[j] = e;
   }
   int v_t[SCAN_V_REGS], v_g[SCAN_V_REGS];
 #pragma unroll
@@ -173,6 +159,26 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
           fk[j] = __fdividef(fk[j], 1.f + __expf(-fk[j]));
           fq[j] = __fdividef(fq[j], 1.f + __expf(-fq[j]));
         }
+        if (RET) {
+          fk[j] *= p.k_scale;
+          const int e = kq_w[j], half = p.rot_dims >> 1;
+          if (e < p.rot_dims) {
+            const bool lower = e < half;
+            const int o = lower ? half : -half;        // the pair's other element
+            const float pk = to_f32(kg[row0 + kq_g[j] + o]) * p.k_scale;
+            const float pq = to_f32(qg[row0 + kq_g[j] + o]) * p.q_scale;
+            float sn, cs;
+            sincosf((float)p.positions[t0 + kq_t[j]] * p.inv_freq[lower ? e : e - half], &sn, &cs);
+            if (lower) sn = -sn;
+            fk[j] = fk[j] * cs + pk * sn;
+            fq[j] = fq[j] * cs + pq * sn;
+          }
+        }
+      }
+      if (GLA) {
+        fw[j] = 0.f;
+        if (kq_t[j] < n && kq_e[j])
+          fw[j] = expf(ra_logsigmoid(wg[(size_t)(t0 + kq_t[j]) * p.ldw + kq_w[j]] + w0[kq_w[j]]) * p.inv_tau);
       }
       if (WKV) {                                     // the decay exp(-exp(z + w0)), float from its pre-activation on
         fw[j] = 0.f;
@@ -193,7 +199,7 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
       if (kq_t[j] < SCAN_CHUNK_MAX) {
         buf[kq_l[j]] = fk[j];
         buf[kq_l[j] + R * PITCH] = fq[j];
-        if (WKV) buf[kq_l[j] + 2 * R * PITCH] = fw[j];
+        if (CHANNEL) buf[kq_l[j] + 2 * R * PITCH] = fw[j];
       }
     }
 #pragma unroll
@@ -205,7 +211,7 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
   };
   float* st = p.state + (size_t)slot * p.slot_stride + (size_t)(head * p.waves_per_head + (active ? w : 0)) * p.wave_floats;
   const bool zero = p.fresh[seq] != 0;
-  const float fade = DECAY ? p.head_decay[head] : 1.f;
+  const float fade = (DECAY || RET) ? p.head_decay[head] : 1.f;
   float S[NPL], nrm[NPL], bonus[NPL];
 #pragma unroll
   for (int i = 0; i < NPL; ++i) {
@@ -225,13 +231,13 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
     const int n = min(CT, last - t0);
     if (active) {
       const int vcol = (tid / RA_WAVE) * CPW + c;
-      struct Operands { float k[NPL], q[NPL], w[WKV ? NPL : 1], v, g0, g1, g2; };
+      struct Operands { float k[NPL], q[NPL], w[CHANNEL ? NPL : 1], v, g0, g1, g2; };
       auto read = [&](int tt, Operands& x) {         // a token's operands out of LDS
         const float* kp = buf + (size_t)tt * NV * R * PITCH + r * PITCH;
         const float* qp = kp + R * PITCH;
 #pragma unroll
         for (int i = 0; i < NPL; ++i) { x.k[i] = kp[i]; x.q[i] = qp[i]; }
-        if (WKV) {
+        if (CHANNEL) {
 #pragma unroll
           for (int i = 0; i < NPL; ++i) x.w[i] = qp[R * PITCH + i];
         }
@@ -266,7 +272,15 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
             S[i] = x.w[i] * S[i] + kv;
           }
           o = group_sum<R>(po[0] + po[1]);
-        } else if (DECAY) {
+        } else if (GLA) {
+          float po[2] = {0.f, 0.f};
+#pragma unroll
+          for (int i = 0; i < NPL; ++i) {
+            S[i] = x.w[i] * S[i] + x.k[i] * x.v;
+            po[i & 1] += S[i] * x.q[i];
+          }
+          o = group_sum<R>(po[0] + po[1]);
+        } else if (DECAY || RET) {
           float po[2] = {0.f, 0.f};
 #pragma unroll
           for (int i = 0; i < NPL; ++i) {
@@ -343,7 +357,7 @@ __global__ __launch_bounds__(256) void matrix_memory_gate_scan_kernel(
       float zf = z[(size_t)t * 2 * H + H + head] + bias[H + head];
       if (cap > 0.f) { zi = cap * tanhf(zi / cap); zf = cap * tanhf(zf / cap); }
       a = zi;
-      b = logsigmoid_f(zf);
+      b = ra_logsigmoid(zf);
     }
     float A = a, B = b;
     sA[tid] = A;
@@ -386,7 +400,7 @@ __global__ void delta_rule_gates_kernel(float* __restrict__ gb, const float* __r
   const int j = (int)(i % (2 * H));
   const float z = gb[i];
   if (j < H) gb[i] = 1.f / (1.f + expf(-z));
-  else gb[i] = expf(-expf(a_log[j - H]) * softplus_f(z + dt_bias[j - H]));
+  else gb[i] = expf(-expf(a_log[j - H]) * ra_softplus(z + dt_bias[j - H]));
 }
 
 // ---------------------------------------------------------------------------
@@ -484,7 +498,7 @@ __global__ void delta_rule_tail_kernel(const TA* __restrict__ proj, int ld, floa
 
 // ---------------------------------------------------------------------------
 // out[t, h, :] = read[t, h, :] / rms(read[t, h, :]) * weight * act(gate[t, h, :]); act = sigmoid or silu;
-// weight is [heads * dv] (w_head_stride = dv) or one [dv] for all heads (0). One wave a (token, head).
+// weight is [heads * dv] (w_head_stride = dv), one [dv] for all heads (0), or absent (null). One wave a (token, head).
 // ---------------------------------------------------------------------------
 template <typename TA>
 __global__ void head_norm_gate_kernel(const float* __restrict__ read, const float* __restrict__ weight,
@@ -506,8 +520,39 @@ __global__ void head_norm_gate_kernel(const float* __restrict__ read, const floa
   for (int e = lane; e < dv; e += RA_WAVE) {
     const float z = to_f32(g[e]);
     const float s = 1.f / (1.f + expf(-z));
-    o[e] = from_f32<TA>(x[e] * rstd * wt[e] * (silu ? z * s : s));
+    o[e] = from_f32<TA>(x[e] * rstd * (weight ? wt[e] : 1.f) * (silu ? z * s : s));
   }
+}
+
+// The same for heads of up to 512 entries, a multiple of 8 that makes a power of two of 8-entry runs: a lane holds one
+// run, 16-byte accesses, a wave 512 / dv heads; the sum stays inside a head's lanes.
+template <typename TA, int LPH>
+__global__ void head_norm_gate_run_kernel(const float* __restrict__ read, const float* __restrict__ weight,
+                                          int w_head_stride, const TA* __restrict__ gate, int ldg, int silu, float eps,
+                                          int H, TA* __restrict__ out, long n_units) {
+  constexpr int dv = LPH * 8;
+  const int ln = threadIdx.x % LPH;
+  const long idx = ((long)blockIdx.x * blockDim.x + threadIdx.x) / LPH;
+  const bool live = idx < n_units;
+  const long at = live ? idx : n_units - 1;              // lanes past the end stay for the exchange of sums
+  const long t = at / H;
+  const int h = (int)(at % H);
+  float x[8], w[8], z[8];
+  Vec8<float>::load(read + (size_t)at * dv + ln * 8, x);
+  Vec8<TA>::load(gate + (size_t)t * ldg + (size_t)h * dv + ln * 8, z);
+  if (weight) Vec8<float>::load(weight + (size_t)h * w_head_stride + ln * 8, w);
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+#pragma unroll
+  for (int m = LPH / 2; m > 0; m >>= 1) ss += __shfl_xor(ss, m, RA_WAVE);
+  const float rstd = 1.f / sqrtf(ss / (float)dv + eps);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float s = 1.f / (1.f + expf(-z[e]));
+    x[e] = x[e] * rstd * (weight ? w[e] : 1.f) * (silu ? z[e] * s : s);
+  }
+  if (live) Vec8<TA>::store(out + (size_t)at * dv + ln * 8, x);
 }
 
 // The same for heads wider than a wave can walk quickly (one "head" as wide as all read-outs together): a workgroup a
@@ -533,7 +578,9 @@ __global__ void head_norm_gate_wide_kernel(const float* __restrict__ read, const
     for (int e = 0; e < 8; ++e) a[r][e] = 0.f;
     if (c >= dv) continue;
     Vec8<float>::load(x + c, a[r]);
-    Vec8<float>::load(wt + c, w[r]);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) w[r][e] = 1.f;
+    if (weight) Vec8<float>::load(wt + c, w[r]);
     Vec8<TA>::load(g + c, z[r]);
 #pragma unroll
     for (int e = 0; e < 8; ++e) ss += a[r][e] * a[r][e];
@@ -811,6 +858,72 @@ extern "C" int ra_decay_scan(const void* proj, int act_dtype, int ld, int q_off,
   return 0;
 }
 
+// kind 3 of ra_scan_state_floats: S <- decays[h] S + k v^T, o = S^T q, q and k turned by their position over their first
+// rot_dims elements (pairs (i, i + rot_dims / 2), angle position * inv_freq[i]; 0: not turned) and times q_scale / k_scale.
+extern "C" int ra_retention_scan(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off,
+                                 const float* decays, const int* positions, const float* inv_freq, int rot_dims,
+                                 float q_scale, float k_scale, float* state, long slot_stride, const int* cu_tokens,
+                                 const int* state_slots, const int* fresh, int n_seqs, int n_tokens, int max_q_len,
+                                 int heads, int key_dim, int value_dim, float* out, hipStream_t stream) {
+  RA_CHECK(n_seqs > 0 && n_tokens > 0 && heads > 0, "retention_scan: %d requests, %d tokens, %d heads", n_seqs, n_tokens, heads);
+  RA_CHECK(decays != nullptr, "retention_scan: one factor a head is needed");
+  RA_CHECK(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= key_dim && (rot_dims == 0 || (positions && inv_freq)),
+           "retention_scan: %d turned elements of %d", rot_dims, key_dim);
+  ScanGeom g;
+  RA_CHECK(scan_geom(3, key_dim, value_dim, &g), "retention_scan: heads of %d x %d (keys up to 512)", key_dim, value_dim);
+  RA_CHECK(slot_stride >= (long)heads * g.waves * g.wave_floats, "retention_scan: a state slot of %ld floats, need %ld",
+           slot_stride, (long)heads * g.waves * g.wave_floats);
+  RA_CHECK(heads <= 65535, "retention_scan: %d heads in one launch", heads);
+  RA_CHECK(act_dtype == RA_F32 || act_dtype == RA_BF16, "retention_scan: unknown dtype tag %d", act_dtype);
+  const ScanLaunch L = scan_launch(g, n_seqs, heads, max_q_len);
+  const size_t es = act_dtype == RA_F32 ? 4 : 2;
+  ScanArgs a = {};
+  a.q = (const char*)proj + (size_t)q_off * es;
+  a.k = (const char*)proj + (size_t)k_off * es;
+  a.v = (const char*)proj + (size_t)v_off * es;
+  a.ld = ld; a.q_heads = heads; a.gates = nullptr; a.state = state; a.slot_stride = slot_stride;
+  a.cu_tokens = cu_tokens; a.state_slots = state_slots; a.fresh = fresh;
+  a.H = heads; a.dk = key_dim; a.dv = value_dim; a.waves_per_head = g.waves; a.wave_floats = g.wave_floats;
+  a.chunk = L.chunk; a.q_scale = q_scale; a.k_scale = k_scale; a.out = out;
+  a.head_decay = decays; a.positions = positions; a.inv_freq = inv_freq; a.rot_dims = rot_dims;
+  if (act_dtype == RA_F32) scan_dispatch<float, SCAN_RETENTION>(g, L, a, stream);
+  else scan_dispatch<bf16_t, SCAN_RETENTION>(g, L, a, stream);
+  RA_LAUNCH_CHECK("retention_scan");
+  return 0;
+}
+
+// kind 4 of ra_scan_state_floats: alpha = sigmoid(z + bias)^(1 / tau) a key channel, S <- diag(alpha) S + k v^T, o = S^T q,
+// q times q_scale. z: float rows of heads * key_dim, ldz apart.
+extern "C" int ra_gla_scan(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off, const float* z, int ldz,
+                           const float* bias, float tau, float q_scale, float* state, long slot_stride,
+                           const int* cu_tokens, const int* state_slots, const int* fresh, int n_seqs, int n_tokens,
+                           int max_q_len, int heads, int key_dim, int value_dim, float* out, hipStream_t stream) {
+  RA_CHECK(n_seqs > 0 && n_tokens > 0 && heads > 0, "gla_scan: %d requests, %d tokens, %d heads", n_seqs, n_tokens, heads);
+  RA_CHECK(z != nullptr && bias != nullptr && ldz >= heads * key_dim && tau > 0.f,
+           "gla_scan: pre-activation rows of %d for %d heads of %d, tau %g", ldz, heads, key_dim, tau);
+  ScanGeom g;
+  RA_CHECK(scan_geom(4, key_dim, value_dim, &g), "gla_scan: heads of %d x %d (keys up to 512)", key_dim, value_dim);
+  RA_CHECK(slot_stride >= (long)heads * g.waves * g.wave_floats, "gla_scan: a state slot of %ld floats, need %ld",
+           slot_stride, (long)heads * g.waves * g.wave_floats);
+  RA_CHECK(heads <= 65535, "gla_scan: %d heads in one launch", heads);
+  RA_CHECK(act_dtype == RA_F32 || act_dtype == RA_BF16, "gla_scan: unknown dtype tag %d", act_dtype);
+  const ScanLaunch L = scan_launch(g, n_seqs, heads, max_q_len, 3);
+  const size_t es = act_dtype == RA_F32 ? 4 : 2;
+  ScanArgs a = {};
+  a.q = (const char*)proj + (size_t)q_off * es;
+  a.k = (const char*)proj + (size_t)k_off * es;
+  a.v = (const char*)proj + (size_t)v_off * es;
+  a.ld = ld; a.q_heads = heads; a.gates = nullptr; a.state = state; a.slot_stride = slot_stride;
+  a.cu_tokens = cu_tokens; a.state_slots = state_slots; a.fresh = fresh;
+  a.H = heads; a.dk = key_dim; a.dv = value_dim; a.waves_per_head = g.waves; a.wave_floats = g.wave_floats;
+  a.chunk = L.chunk; a.q_scale = q_scale; a.out = out;
+  a.w = z; a.ldw = ldz; a.w0 = bias; a.inv_tau = 1.f / tau;
+  if (act_dtype == RA_F32) scan_dispatch<float, SCAN_GLA>(g, L, a, stream);
+  else scan_dispatch<bf16_t, SCAN_GLA>(g, L, a, stream);
+  RA_LAUNCH_CHECK("gla_scan");
+  return 0;
+}
+
 extern "C" int ra_head_norm_gate(const float* read, const float* weight, int per_head_weight, const void* gate,
                                  int ldg, int act_dtype, int silu, float eps, int n_tokens, int heads, int value_dim,
                                  void* out, hipStream_t stream) {
@@ -832,6 +945,31 @@ extern "C" int ra_head_norm_gate(const float* read, const float* weight, int per
       head_norm_gate_wide_kernel<bf16_t><<<(unsigned)units, threads, 0, stream>>>(read, weight, ws, (const bf16_t*)gate,
                                                                                   ldg, silu, eps, heads, value_dim,
                                                                                   (bf16_t*)out);
+    RA_LAUNCH_CHECK("head_norm_gate");
+    return 0;
+  }
+  const int runs = value_dim / 8;
+  if (value_dim % 8 == 0 && runs <= RA_WAVE && (runs & (runs - 1)) == 0 && ((uintptr_t)read % 16) == 0 &&
+      ((uintptr_t)weight % 16) == 0 && ((uintptr_t)gate % 16) == 0 && ((long)ldg * es) % 16 == 0 &&
+      ((uintptr_t)out % 16) == 0 && (act_dtype == RA_F32 || act_dtype == RA_BF16)) {
+    const unsigned grid = (unsigned)((units * runs + 255) / 256);
+#define RA_HNG(L)                                                                                                        \
+  do {                                                                                                                   \
+    if (act_dtype == RA_F32)                                                                                             \
+      head_norm_gate_run_kernel<float, L><<<grid, 256, 0, stream>>>(read, weight, ws, (const float*)gate, ldg, silu, eps, \
+                                                                    heads, (float*)out, units);                          \
+    else                                                                                                                 \
+      head_norm_gate_run_kernel<bf16_t, L><<<grid, 256, 0, stream>>>(read, weight, ws, (const bf16_t*)gate, ldg, silu,   \
+                                                                     eps, heads, (bf16_t*)out, units);                   \
+  } while (0)
+    if (runs == 1) RA_HNG(1);
+    else if (runs == 2) RA_HNG(2);
+    else if (runs == 4) RA_HNG(4);
+    else if (runs == 8) RA_HNG(8);
+    else if (runs == 16) RA_HNG(16);
+    else if (runs == 32) RA_HNG(32);
+    else RA_HNG(64);
+#undef RA_HNG
     RA_LAUNCH_CHECK("head_norm_gate");
     return 0;
   }

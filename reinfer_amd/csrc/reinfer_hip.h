@@ -5,7 +5,7 @@
 #pragma once
 #include <hip/hip_runtime.h>
 
-#define RA_ABI_VERSION 23
+#define RA_ABI_VERSION 24
 
 #ifdef __cplusplus
 extern "C" {
@@ -29,7 +29,8 @@ int ra_add_group_rmsnorm(float* resid, const void* delta, const void* weight, in
 int ra_qk_norm_rope_cache(void* qkv, int act_dtype, const void* q_weight, const void* k_weight,
                           int weight_dtype, float eps, const int* positions, const float* inv_freq,
                           int rotary_dim, int rope_style, const int* slots, void* kcache, void* vcache,
-                          int block_size, int n_tokens, int Hq, int Hkv, int d, hipStream_t stream);
+                          int block_size, int n_tokens, int Hq, int Hkv, int d, int values_are_keys,
+                          hipStream_t stream);
 // The same from the partial results of ra_gemm_wide_partial (added here, in range order), optionally scaled
 // by the RMSNorm that product carried (in_ss [in_parts][n_tokens], eps, width); the rotated q goes to q_out.
 int ra_qk_norm_rope_cache_sums(const float* parts, int n_ranges, const float* in_ss, int in_parts, float in_eps,
@@ -37,7 +38,8 @@ int ra_qk_norm_rope_cache_sums(const float* parts, int n_ranges, const float* in
                                const void* k_weight, int weight_dtype, float eps, const int* positions,
                                const float* inv_freq, int rotary_dim, int rope_style, const int* slots,
                                void* kcache, void* vcache, int block_size, int n_tokens, int Hq, int Hkv, int d,
-                               hipStream_t stream);
+                               int values_are_keys, hipStream_t stream);
+// values_are_keys: rows hold q and k heads alone, (Hq + Hkv) * d, and the cached value is the key before its norm
 
 // gate_up is [T, 2I]: group == 0: gate columns [0, I), up columns [I, 2I); group > 0: gate and
 // up interleaved in runs of `group` columns (gate run, then the up run of the same features)
@@ -54,11 +56,12 @@ int ra_attention_plain(const void* q, int q_stride, void* out, int out_stride, c
                        int Hq, int Hkv, int d, float scale, int window, hipStream_t stream);
 // The `_mod` forms of the three attention kernels change a score between the scaled product and the softmax:
 // softcap > 0: s <- softcap tanh(s / softcap); r1, r2 (float, one entry a query head, both or neither):
-// s <- s - r1[h] ln(1 + r2[h] (query position - key position)); the cap first.
+// s <- s - r1[h] ln(1 + r2[h] (query position - key position)); the cap first. keep > 0 with a window: the request's
+// first keep keys are seen as well, however far the window has moved on.
 int ra_attention_plain_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                            const void* vcache, int act_dtype, const int* block_tables, int max_blocks,
                            const int* token_list, const int* seq_of_token, const int* positions, int n_tokens,
-                           int block_size, int Hq, int Hkv, int d, float scale, int window, float softcap,
+                           int block_size, int Hq, int Hkv, int d, float scale, int window, int keep, float softcap,
                            const float* r1, const float* r2, hipStream_t stream);
 // act 2 of ra_act_mul with its bound: g <- min(g, lim), u <- clamp(u, -lim, lim), out = g sigmoid(1.702 g) (u + 1)
 int ra_act_mul_bounded(const void* gate_up, void* out, int act_dtype, int n_tokens, int intermediate, int group,
@@ -133,7 +136,7 @@ int ra_attention_decode(const void* q, int q_stride, void* out, int out_stride, 
 int ra_attention_decode_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                             const void* vcache, const int* block_tables, int max_blocks,
                             const int* token_list, const int* seq_of_token, const int* positions,
-                            int n_tokens, int block_size, int Hq, int Hkv, int d, float scale, int window,
+                            int n_tokens, int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
                             int chunk, int max_chunks, int waves, float* part_o, float* part_ml, float softcap,
                             const float* r1, const float* r2, hipStream_t stream);
 int ra_attention_prefill_supports(int Hq, int Hkv, int d, int block_size);
@@ -157,12 +160,12 @@ int ra_attention_prefill_split(const void* q, int q_stride, void* out, int out_s
 
 int ra_attention_prefill_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                              const void* vcache, const int* block_tables, int max_blocks, const int* tile_info,
-                             int n_tiles, int block_size, int Hq, int Hkv, int d, float scale, int window,
+                             int n_tiles, int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
                              float softcap, const float* r1, const float* r2, hipStream_t stream);
 int ra_attention_prefill_split_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                                    const void* vcache, const int* block_tables, int max_blocks, const int* tile_info,
                                    int n_tiles, const int* ranges, const int* merge_info, int n_merge, float* part_o,
-                                   float* part_ml, int block_size, int Hq, int Hkv, int d, float scale, int window,
+                                   float* part_ml, int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
                                    float softcap, const float* r1, const float* r2, hipStream_t stream);
 
 int ra_sample_slices(int vocab);
@@ -309,6 +312,33 @@ int ra_gemm_skinny_scaled(const void* A, const void* W, float* C, int M, int N, 
                           float acc_scale, hipStream_t stream);
 int ra_gemm_wide_scaled(const void* A, const void* W, float* C, int M, int N, int K, int lda, int ldc, float* scratch,
                         long scratch_floats, float acc_scale, hipStream_t stream);
+
+// Retention: S <- decays[h] S + k v^T, o = S^T q, q and k turned by their position over their first rot_dims elements
+// (pairs (i, i + rot_dims / 2), angle position * inv_freq[i]), times q_scale and k_scale. State: ra_scan_state_floats kind 3.
+int ra_retention_scan(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off, const float* decays,
+                      const int* positions, const float* inv_freq, int rot_dims, float q_scale, float k_scale, float* state,
+                      long slot_stride, const int* cu_tokens, const int* state_slots, const int* fresh, int n_seqs,
+                      int n_tokens, int max_q_len, int heads, int key_dim, int value_dim, float* out, hipStream_t stream);
+// Gated linear attention: alpha = sigmoid(z + bias)^(1 / tau) a key channel; S <- diag(alpha) S + k v^T, o = S^T q. Kind 4.
+int ra_gla_scan(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off, const float* z, int ldz,
+                const float* bias, float tau, float q_scale, float* state, long slot_stride, const int* cu_tokens,
+                const int* state_slots, const int* fresh, int n_seqs, int n_tokens, int max_q_len, int heads, int key_dim,
+                int value_dim, float* out, hipStream_t stream);
+// The same recurrences (silu: ra_decay_scan's) in chunks of 16 tokens on the float matrix cores, keys up to 256, from and
+// into the same state. Scratch: turn n_tokens * rot_dims floats; cum n_tokens * heads * key_dim floats.
+int ra_decay_chunks(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off, int silu, const float* decays,
+                    const int* positions, const float* inv_freq, int rot_dims, float* turn, float q_scale, float k_scale,
+                    float* state, long slot_stride, const int* cu_tokens, const int* state_slots, const int* fresh,
+                    int n_seqs, int n_tokens, int heads, int key_dim, int value_dim, float* out, hipStream_t stream);
+int ra_gla_chunks(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off, const float* z, int ldz,
+                  const float* bias, float tau, float* cum, float q_scale, float* state, long slot_stride,
+                  const int* cu_tokens, const int* state_slots, const int* fresh, int n_seqs, int n_tokens, int max_q_len,
+                  int heads, int key_dim, int value_dim, float* out, hipStream_t stream);
+// Several residual streams: X_t <- sum_s mix[s, t] X_s + w_out[t] y (y null: as they are; base: every stream is this row),
+// u = sum_t w_in[t] X_t (null: ones); out = u / sqrt(mean u^2 + eps) * weight (weight null: u). store: keep the new streams.
+int ra_hyper_step(float* streams, const float* base, const void* y, int y_dtype, const float* mix, const float* w_out,
+                  const float* w_in, const float* weight, float eps, const int* rows, int n_rows, int n_streams, int hidden,
+                  int store, void* out, int out_dtype, hipStream_t stream);
 
 // ---- recurrent mixers (recurrent.hip) ----
 // floats of state a request slot holds for the scan kernels; kind 0: matrix memory, 1: delta rule, 2: wkv, 3: a memory

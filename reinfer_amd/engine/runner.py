@@ -58,14 +58,17 @@ class ModelRunner:
 
         # which run-order entries keep keys of their own, and with which window
         windows: List[Optional[int]] = []
+        keeps: List[int] = []
         for e, need in zip(spec.run_order, needs):
             if paged_need(need) is not None and e.cache_from is None:
                 windows.append(paged_need(need).window)
+                keeps.append(int(getattr(paged_need(need), "keep", 0)))
             else:
                 windows.append(None)
+                keeps.append(0)
         # no layer with keys of its own: no group, no pool, no block tables; requests then hold a state
         # slot each and are admitted by slots alone
-        groups = plan_groups(windows)
+        groups = plan_groups(windows, keeps)
         self.groups = groups
         group_of = {i: g for g, gs in enumerate(groups) for i in gs.entries}
 

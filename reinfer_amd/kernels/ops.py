@@ -105,10 +105,12 @@ class HipKernels:
                            k_weight: Optional[torch.Tensor], eps: float, positions: torch.Tensor,
                            inv_freq: torch.Tensor, rotary_dim: int, rope_style: int,
                            slots: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
-                           num_heads: int, num_kv_heads: int, head_dim: int) -> None:
+                           num_heads: int, num_kv_heads: int, head_dim: int, values_are_keys: bool = False) -> None:
+        """Head norm and rotation of q (in place) and k, k and v into the cache. ``values_are_keys``: the rows hold
+        q and k alone, and the value that is cached is the key as it stands there, before norm and rotation."""
         _dev(qkv, q_weight, k_weight, positions, inv_freq, slots, kcache, vcache)
         T = qkv.shape[0]
-        width = (num_heads + 2 * num_kv_heads) * head_dim
+        width = (num_heads + (1 if values_are_keys else 2) * num_kv_heads) * head_dim
         if qkv.shape != (T, width) or not qkv.is_contiguous():
             raise ValueError(f"qk_norm_rope_cache: qkv {tuple(qkv.shape)}, expected [T, {width}] contiguous")
         self._check_cache("qk_norm_rope_cache", kcache, vcache, num_kv_heads, head_dim)
@@ -129,7 +131,8 @@ class HipKernels:
         library.call("ra_qk_norm_rope_cache", qkv.data_ptr(), _tag(qkv, "qkv"), _ptr(q_weight),
                      _ptr(k_weight), wtag, float(eps), positions.data_ptr(), inv_freq.data_ptr(),
                      int(rotary_dim), int(rope_style), slots.data_ptr(), kcache.data_ptr(),
-                     vcache.data_ptr(), kcache.shape[2] * 16, T, num_heads, num_kv_heads, head_dim, _stream())
+                     vcache.data_ptr(), kcache.shape[2] * 16, T, num_heads, num_kv_heads, head_dim,
+                     1 if values_are_keys else 0, _stream())
 
     # ---- the q/k/v product left in K ranges for the kernel that consumes it
     def linear_ranges(self, x: torch.Tensor, weight: torch.Tensor):
@@ -192,7 +195,7 @@ class HipKernels:
                      int(in_width), q_out.data_ptr(), q_out.stride(0), _tag(q_out, "q"), _ptr(q_weight),
                      _ptr(k_weight), wtag, float(eps), positions.data_ptr(), inv_freq.data_ptr(),
                      int(rotary_dim), int(rope_style), slots.data_ptr(), kcache.data_ptr(), vcache.data_ptr(),
-                     kcache.shape[2] * 16, T, num_heads, num_kv_heads, head_dim, _stream())
+                     kcache.shape[2] * 16, T, num_heads, num_kv_heads, head_dim, 0, _stream())
 
     GATE_ACTS = {"silu": 0, "gelu_tanh": 1, "swish_bounded": 2}
 
@@ -221,12 +224,14 @@ class HipKernels:
 
     def attention(self, q: torch.Tensor, q_stride: int, out: torch.Tensor, kcache: torch.Tensor,
                   vcache: torch.Tensor, batch, num_heads: int, num_kv_heads: int, head_dim: int,
-                  scale: float, window: int, group: int, softcap: float = 0.0, distance=None) -> None:
+                  scale: float, window: int, group: int, softcap: float = 0.0, distance=None,
+                  keep: int = 0) -> None:
         """Attention of every token of the step over its request's cache.
 
         ``softcap`` > 0: score <- softcap * tanh(score / softcap); ``distance`` = (r1, r2), two float32 vectors
         with one entry a query head: score <- score - r1[h] * ln(1 + r2[h] * (query position - key position)),
-        behind the cap. Every kernel below applies them alike.
+        behind the cap. ``keep`` > 0 with a window: a request's first ``keep`` keys are seen as well, however far
+        the window has moved on. Every kernel below applies them alike.
 
         ``q`` is the buffer whose row ``t`` holds the query heads of token t at
         its start (row stride ``q_stride`` elements); ``batch`` is the step's
@@ -240,6 +245,10 @@ class HipKernels:
         mod = self._score_mod(softcap, distance, num_heads, q.device)
         # handed on only where there is a change, so that the kernels' callers of old need not know of it
         changed = {"mod": mod} if (mod[0] > 0.0 or mod[1] is not None) else {}
+        if keep < 0:
+            raise ValueError("attention: a negative number of kept keys")
+        if keep and window:
+            changed["keep"] = int(keep)
         if q.dtype != torch.bfloat16:
             return self.attention_plain(q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads,
                                         head_dim, scale, window, group, **changed)
@@ -517,7 +526,7 @@ class HipKernels:
         return tables
 
     def attention_plain(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
-                        scale, window, group, token_list=None, n_listed=None, mod=(0.0, None, None)) -> None:
+                        scale, window, group, token_list=None, n_listed=None, mod=(0.0, None, None), keep: int = 0) -> None:
         tables = self._check_attention(q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads,
                                        head_dim, group)
         n = batch.num_tokens if token_list is None else int(n_listed)
@@ -525,7 +534,7 @@ class HipKernels:
                      kcache.data_ptr(), vcache.data_ptr(), _tag(q, "attention"), tables.data_ptr(),
                      tables.shape[1], _ptr(token_list), batch.seq_of_token.data_ptr(),
                      batch.positions.data_ptr(), n, kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim,
-                     float(scale), int(window), mod[0], mod[1], mod[2], _stream())
+                     float(scale), int(window), int(keep), mod[0], mod[1], mod[2], _stream())
 
     # The decode kernel runs in workgroups of 12 waves from this many (token, KV head) pairs on, or over
     # contexts longer than this; below both, in workgroups of 4 (measured with 32 query heads over 8 KV
@@ -582,13 +591,16 @@ class HipKernels:
 
     def attention_decode(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
                          scale, window, group, token_list=None, n_listed=None, max_ctx=None,
-                         chunk=None, waves=None, mod=(0.0, None, None)) -> None:
+                         chunk=None, waves=None, mod=(0.0, None, None), keep: int = 0) -> None:
         tables = self._check_attention(q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads,
                                        head_dim, group)
         if q.dtype != torch.bfloat16:
             raise TypeError("attention_decode: bfloat16 only")
         n = batch.num_tokens if token_list is None else int(n_listed)
         max_ctx = int(max_ctx or batch.max_ctx_len)
+        if window > 0:
+            # no token reads more than its window (from the tile that holds its first key) and the kept keys' tiles
+            max_ctx = min(max_ctx, int(window) + 15 + -(-int(keep) // 16) * 16)
         if chunk is None:
             chunk, max_chunks, waves = self.decode_chunk(n, num_heads, num_kv_heads, head_dim, max_ctx)
         else:
@@ -605,13 +617,13 @@ class HipKernels:
         library.call("ra_attention_decode_mod", q.data_ptr(), q_stride, out.data_ptr(), out.stride(0),
                      kcache.data_ptr(), vcache.data_ptr(), tables.data_ptr(), tables.shape[1],
                      _ptr(token_list), None if one_each else batch.seq_of_token.data_ptr(), batch.positions.data_ptr(), n,
-                     kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim, float(scale), int(window),
+                     kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim, float(scale), int(window), int(keep),
                      int(chunk), int(max_chunks), int(waves), _ptr(part_o), _ptr(part_ml), mod[0], mod[1], mod[2],
                      _stream())
 
     def attention_prefill(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
                           scale, window, group, tiles, n_tiles, ranges=None, merge=None, n_merge: int = 0,
-                          n_slots: int = 0, mod=(0.0, None, None)) -> None:
+                          n_slots: int = 0, mod=(0.0, None, None), keep: int = 0) -> None:
         """``tiles``: four ints a listed query tile (request row, first token row, queries, first
         position). With ``ranges`` (three ints a listed tile: first key, one past the last, the part's
         slot or -1) some tiles are listed in several parts by keys, and ``merge`` (four ints a cut tile:
@@ -635,12 +647,12 @@ class HipKernels:
                          kcache.data_ptr(), vcache.data_ptr(), tables.data_ptr(), tables.shape[1],
                          tiles.data_ptr(), int(n_tiles), ranges.data_ptr(), merge.data_ptr(), int(n_merge),
                          part_o.data_ptr(), part_ml.data_ptr(), kcache.shape[2] * 16, num_heads, num_kv_heads,
-                         head_dim, float(scale), int(window), mod[0], mod[1], mod[2], _stream())
+                         head_dim, float(scale), int(window), int(keep), mod[0], mod[1], mod[2], _stream())
             return
         library.call("ra_attention_prefill_mod", q.data_ptr(), q_stride, out.data_ptr(), out.stride(0),
                      kcache.data_ptr(), vcache.data_ptr(), tables.data_ptr(), tables.shape[1],
                      tiles.data_ptr(), int(n_tiles), kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim,
-                     float(scale), int(window), mod[0], mod[1], mod[2], _stream())
+                     float(scale), int(window), int(keep), mod[0], mod[1], mod[2], _stream())
 
     # ---------------------------------------------------------------- linear
     def linear(self, x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor,
@@ -1025,7 +1037,7 @@ class HipKernels:
                      1 if gate_per_head else 0, _tag(x, "head_linear"), T, H, N, K, _stream())
 
     # ------------------------------------------------------ recurrent mixers
-    _SCAN_KINDS = {"matrix_memory": 0, "delta_rule": 1, "wkv": 2, "decay_memory": 3}
+    _SCAN_KINDS = {"matrix_memory": 0, "delta_rule": 1, "wkv": 2, "decay_memory": 3, "gated_linear": 4}
 
     def scan_state_floats(self, kind: str, heads: int, key_dim: int, value_dim: int) -> int:
         """Floats of a request's state slot that the scan kernel of ``kind`` ("matrix_memory", "delta_rule", "wkv")
@@ -1209,17 +1221,18 @@ class HipKernels:
             raise ValueError("tanh_rows: a contiguous tensor")
         library.call("ra_tanh_rows", x.data_ptr(), _tag(x, "tanh_rows"), x.numel(), _stream())
 
-    def head_norm_gate(self, read: torch.Tensor, weight: torch.Tensor, per_head: bool, gate: torch.Tensor, kind: str,
+    def head_norm_gate(self, read: torch.Tensor, weight: Optional[torch.Tensor], per_head: bool, gate: torch.Tensor, kind: str,
                        eps: float, heads: int, value_dim: int, out: torch.Tensor) -> None:
         """out[t, h] = read[t, h] / rms(read[t, h]) * weight * act(gate[t, h]) head by head: ``read`` float32
         [T, heads * value_dim], ``weight`` float32 [heads * value_dim] (``per_head``) or [value_dim] for all
-        heads, ``gate`` [T, >= heads * value_dim] rows of the activations' dtype, ``kind`` "sigmoid" or "silu"."""
+        heads or None, ``gate`` [T, >= heads * value_dim] rows of the activations' dtype, ``kind`` "sigmoid" or "silu"."""
         _dev(read, weight, gate, out)
         T = read.shape[0]
         n = heads * value_dim
         if read.shape != (T, n) or read.dtype != torch.float32 or not read.is_contiguous():
             raise ValueError(f"head_norm_gate: read is contiguous float32 [T, {n}]")
-        if weight.dtype != torch.float32 or weight.shape != ((n,) if per_head else (value_dim,)) or not weight.is_contiguous():
+        if weight is not None and (weight.dtype != torch.float32 or not weight.is_contiguous()
+                                   or weight.shape != ((n,) if per_head else (value_dim,))):
             raise ValueError(f"head_norm_gate: weight {tuple(weight.shape)} {weight.dtype}")
         if gate.dim() != 2 or gate.shape[0] != T or gate.shape[1] < n or gate.stride(1) != 1 or gate.dtype != out.dtype:
             raise ValueError(f"head_norm_gate: gate {tuple(gate.shape)}, expected rows of at least {n} in the output's dtype")
@@ -1227,7 +1240,7 @@ class HipKernels:
             raise ValueError(f"head_norm_gate: out is contiguous [T, {n}]")
         if kind not in ("sigmoid", "silu"):
             raise ValueError(f"head_norm_gate: gate kind {kind!r}")
-        library.call("ra_head_norm_gate", read.data_ptr(), weight.data_ptr(), 1 if per_head else 0, gate.data_ptr(),
+        library.call("ra_head_norm_gate", read.data_ptr(), _ptr(weight), 1 if per_head else 0, gate.data_ptr(),
                      gate.stride(0), _tag(out, "head_norm_gate"), 1 if kind == "silu" else 0, float(eps), T, int(heads),
                      int(value_dim), out.data_ptr(), _stream())
 
@@ -1306,25 +1319,123 @@ class HipKernels:
                      int(width), int(style), _ptr(positions), _ptr(inv_freq), float(sign), _ptr(gate),
                      gate.stride(0) if gate is not None else 0, int(gate_stride), _stream())
 
+    # Portions from this many tokens on are taken in chunks of 16 tokens (keys up to CHUNK_KEYS), shorter ones token by
+    # token; either form goes on from the state that the other left.
+    CHUNK_FROM = 17
+    CHUNK_KEYS = 256
+
+    @staticmethod
+    def _check_linear_scan(what: str, proj, q_off, k_off, v_off, heads, key_dim, value_dim, out) -> None:
+        T = proj.shape[0]
+        if proj.dim() != 2 or proj.stride(1) != 1 or max(q_off, k_off) + heads * key_dim > proj.shape[1] \
+                or v_off + heads * value_dim > proj.shape[1] or min(q_off, k_off, v_off) < 0:
+            raise ValueError(f"{what}: the projection rows do not hold q, k and v at the given offsets")
+        if out.shape != (T, heads * value_dim) or out.dtype != torch.float32 or not out.is_contiguous():
+            raise ValueError(f"{what}: out is contiguous float32 [T, {heads * value_dim}]")
+
     def decay_scan(self, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, decays: torch.Tensor,
-                   state: torch.Tensor, batch, heads: int, key_dim: int, value_dim: int, out: torch.Tensor) -> None:
-        """S <- decays[h] S + k v^T, o = S^T q head by head and token by token, q, k and v being the silu of
-        ``proj``'s columns at the given offsets; the state [slots, floats] is float32, ``out`` float32
-        [T, heads * value_dim]."""
-        _dev(proj, decays, state, out)
+                   state: torch.Tensor, batch, heads: int, key_dim: int, value_dim: int, out: torch.Tensor,
+                   act: str = "silu", inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0,
+                   q_scale: float = 1.0, k_scale: float = 1.0, chunks: Optional[bool] = None) -> None:
+        """S <- decays[h] S + k v^T, o = S^T q head by head; the state [slots, floats] is float32, ``out`` float32
+        [T, heads * value_dim]. q, k and v are ``proj``'s columns at the given offsets: with ``act`` "silu" their silu;
+        with "none" as they are, q and k turned by their position over their first ``rot_dims`` elements (pairs
+        (i, i + rot_dims / 2), angle position * inv_freq[i]) and times ``q_scale`` and ``k_scale``. Everything behind
+        the projection is float. ``chunks`` forces the form (None: by the step's longest portion)."""
+        _dev(proj, decays, state, out, inv_freq)
         T = proj.shape[0]
         self._check_scan("decay_scan", state, batch, T)
         if decays.dtype != torch.float32 or decays.shape != (heads,) or not decays.is_contiguous():
             raise ValueError(f"decay_scan: one float32 factor a head ({heads})")
-        if proj.dim() != 2 or proj.stride(1) != 1 or max(q_off, k_off) + heads * key_dim > proj.shape[1] \
-                or v_off + heads * value_dim > proj.shape[1]:
-            raise ValueError("decay_scan: the projection rows do not hold q, k and v at the given offsets")
-        if out.shape != (T, heads * value_dim) or out.dtype != torch.float32 or not out.is_contiguous():
-            raise ValueError(f"decay_scan: out is contiguous float32 [T, {heads * value_dim}]")
-        library.call("ra_decay_scan", proj.data_ptr(), _tag(proj, "decay_scan"), proj.stride(0), int(q_off), int(k_off),
-                     int(v_off), decays.data_ptr(), state.data_ptr(), state.stride(0), batch.cu_tokens.data_ptr(),
-                     batch.state_slots.data_ptr(), batch.fresh.data_ptr(), batch.num_seqs, T, int(batch.max_q_len),
-                     int(heads), int(key_dim), int(value_dim), out.data_ptr(), _stream())
+        self._check_linear_scan("decay_scan", proj, q_off, k_off, v_off, heads, key_dim, value_dim, out)
+        if act not in ("silu", "none"):
+            raise ValueError(f"decay_scan: activation {act!r}; built: silu, none")
+        if act == "silu" and (rot_dims or q_scale != 1.0 or k_scale != 1.0):
+            raise ValueError("decay_scan: with silu q and k neither turn nor carry a factor")
+        if rot_dims < 0 or rot_dims % 2 or rot_dims > key_dim or \
+                (rot_dims and (inv_freq is None or inv_freq.dtype != torch.float32 or inv_freq.numel() < rot_dims // 2
+                               or not inv_freq.is_contiguous())):
+            raise ValueError(f"decay_scan: {rot_dims} turned elements of {key_dim}, float32 frequencies of their pairs")
+        if rot_dims:
+            _int32(batch.positions, "positions", T)
+        tag, longest = _tag(proj, "decay_scan"), int(batch.max_q_len)
+        if chunks is None:
+            chunks = longest >= self.CHUNK_FROM and key_dim <= self.CHUNK_KEYS
+        tail = (state.data_ptr(), state.stride(0), batch.cu_tokens.data_ptr(), batch.state_slots.data_ptr(),
+                batch.fresh.data_ptr(), batch.num_seqs, T)
+        turned = (batch.positions.data_ptr() if rot_dims else None, _ptr(inv_freq) if rot_dims else None, int(rot_dims))
+        if chunks:
+            turn = torch.empty(T * rot_dims, dtype=torch.float32, device=proj.device) if rot_dims else None
+            library.call("ra_decay_chunks", proj.data_ptr(), tag, proj.stride(0), int(q_off), int(k_off), int(v_off),
+                         1 if act == "silu" else 0, decays.data_ptr(), *turned, _ptr(turn), float(q_scale), float(k_scale),
+                         *tail, int(heads), int(key_dim), int(value_dim), out.data_ptr(), _stream())
+        elif act == "silu":
+            library.call("ra_decay_scan", proj.data_ptr(), tag, proj.stride(0), int(q_off), int(k_off), int(v_off),
+                         decays.data_ptr(), *tail, longest, int(heads), int(key_dim), int(value_dim), out.data_ptr(),
+                         _stream())
+        else:
+            library.call("ra_retention_scan", proj.data_ptr(), tag, proj.stride(0), int(q_off), int(k_off), int(v_off),
+                         decays.data_ptr(), *turned, float(q_scale), float(k_scale), *tail, longest, int(heads),
+                         int(key_dim), int(value_dim), out.data_ptr(), _stream())
+
+    def gated_linear_scan(self, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, z: torch.Tensor,
+                          bias: torch.Tensor, tau: float, state: torch.Tensor, batch, heads: int, key_dim: int,
+                          value_dim: int, out: torch.Tensor, q_scale: float = 1.0, chunks: Optional[bool] = None) -> None:
+        """S <- diag(alpha) S + k v^T, o = S^T q head by head with alpha = sigmoid(z + bias)^(1 / tau), one factor a head
+        and key channel (``z`` float32 [T, heads * key_dim], ``bias`` float32 [heads * key_dim]); q times ``q_scale``.
+        State, ``out`` and ``chunks`` as for :meth:`decay_scan`."""
+        _dev(proj, z, bias, state, out)
+        T, n = proj.shape[0], heads * key_dim
+        self._check_scan("gated_linear_scan", state, batch, T)
+        self._check_linear_scan("gated_linear_scan", proj, q_off, k_off, v_off, heads, key_dim, value_dim, out)
+        if z.dim() != 2 or z.shape[0] != T or z.shape[1] < n or z.dtype != torch.float32 or z.stride(1) != 1 \
+                or bias.shape != (n,) or bias.dtype != torch.float32 or not bias.is_contiguous():
+            raise ValueError(f"gated_linear_scan: pre-activations float32 [T, {n}], their bias float32 [{n}]")
+        if not tau > 0.0:
+            raise ValueError("gated_linear_scan: tau is positive")
+        tag, longest = _tag(proj, "gated_linear_scan"), int(batch.max_q_len)
+        if chunks is None:
+            chunks = longest >= self.CHUNK_FROM and key_dim <= self.CHUNK_KEYS
+        head = (proj.data_ptr(), tag, proj.stride(0), int(q_off), int(k_off), int(v_off), z.data_ptr(), z.stride(0),
+                bias.data_ptr(), float(tau))
+        tail = (float(q_scale), state.data_ptr(), state.stride(0), batch.cu_tokens.data_ptr(),
+                batch.state_slots.data_ptr(), batch.fresh.data_ptr(), batch.num_seqs, T, longest, int(heads), int(key_dim),
+                int(value_dim), out.data_ptr(), _stream())
+        if chunks:
+            cum = torch.empty((T, n), dtype=torch.float32, device=proj.device)
+            library.call("ra_gla_chunks", *head, cum.data_ptr(), *tail)
+        else:
+            library.call("ra_gla_scan", *head, *tail)
+
+    # -------------------------------------------------------------- several residual streams
+    def hyper_step(self, streams: torch.Tensor, base: Optional[torch.Tensor], y: Optional[torch.Tensor],
+                   mix: Optional[torch.Tensor], w_out: Optional[torch.Tensor], w_in: Optional[torch.Tensor],
+                   weight: Optional[torch.Tensor], eps: float, out: Optional[torch.Tensor],
+                   rows: Optional[torch.Tensor] = None, store: bool = True) -> None:
+        """``streams`` float32 [T, n, width]: X_t <- sum_s mix[s, t] X_s + w_out[t] y (``y`` None: as they are),
+        u = sum_t w_in[t] X_t (None: ones), ``out`` = u / sqrt(mean u^2 + eps) * weight (``weight`` None: u itself).
+        ``base`` [T, width]: every stream is still this row. ``store``: the new streams are kept; with ``rows`` only
+        those rows are computed, into a compact ``out``, and nothing is kept."""
+        _dev(streams, base, y, mix, w_out, w_in, weight, out, rows)
+        if streams.dim() != 3 or streams.dtype != torch.float32 or not streams.is_contiguous():
+            raise TypeError("hyper_step: the streams are contiguous float32 [T, n, width]")
+        T, n, h = streams.shape
+        for t, shape, what in ((base, (T, h), "base"), (mix, (n, n), "mix"), (w_out, (n,), "out factors"),
+                               (w_in, (n,), "in factors"), (weight, (h,), "norm weight")):
+            if t is not None and (t.dtype != torch.float32 or t.shape != shape or not t.is_contiguous()):
+                raise ValueError(f"hyper_step: {what} {tuple(t.shape)} {t.dtype}, expected contiguous float32 {list(shape)}")
+        if y is not None and (y.shape != (T, h) or not y.is_contiguous() or mix is None or w_out is None):
+            raise ValueError("hyper_step: y is contiguous [T, width] and enters by mix and w_out")
+        n_rows = T
+        if rows is not None:
+            n_rows = rows.numel()
+            _int32(rows, "hyper_step rows", n_rows)
+            store = False
+        if out is not None and (out.shape != (n_rows, h) or not out.is_contiguous()):
+            raise ValueError(f"hyper_step: out {tuple(out.shape)}, expected contiguous [{n_rows}, {h}]")
+        library.call("ra_hyper_step", streams.data_ptr(), _ptr(base), _ptr(y), _tag(y, "hyper_step y") if y is not None else 0,
+                     _ptr(mix), _ptr(w_out), _ptr(w_in), _ptr(weight), float(eps), _ptr(rows), n_rows, n, h,
+                     1 if store else 0, _ptr(out), _tag(out, "hyper_step out") if out is not None else 0, _stream())
 
     def moe_table_route(self, token_ids: torch.Tensor, table: torch.Tensor, ids: torch.Tensor,
                         weights: torch.Tensor) -> None:

@@ -41,7 +41,8 @@ _OTHER = {"latent_prep": "latent norm + rotation + cache write", "head_linear": 
           "rows_rmsnorm": "row norm", "tanh_rows": "tanh", "moe_identity_add": "identity experts",
           "stream_cast": "stream as operand", "sum_norm_add": "sum + norm + stream add",
           "span_rmsnorm": "projection norm", "turn_heads": "turn of heads (+ gate)", "decay_scan": "decay scan",
-          "moe_table_route": "router"}
+          "moe_table_route": "router", "gated_linear_scan": "gated linear scan",
+          "hyper_step": "streams + norm"}
 
 
 class TimedKernels:

@@ -10,7 +10,7 @@ import torch
 
 from .. import kernels
 from ..config.schema import ModelSpec
-from ..parts import KVNeed, LayerCache, StateNeed, lookup
+from ..parts import KVNeed, LayerCache, StateNeed, StreamMix, lookup
 from ..weights import MATRIX, ParamDecl
 
 
@@ -133,6 +133,11 @@ class DecoderModel:
             observer(0, resid.clone())
         embedded = resid.clone() if self.keeps_embedding else None
         delta = None
+        if self.spec.streams:
+            # several streams: all equal to the embedding until the first sublayer's result has entered
+            delta = StreamMix(base=resid)
+            resid = torch.empty((batch.num_tokens, self.spec.streams, self.spec.hidden), dtype=torch.float32,
+                                device=self.device)
         n = len(self.run_order)
         for i, e in enumerate(self.run_order):
             block = self.blocks[e.block]
@@ -156,6 +161,9 @@ class DecoderModel:
                 delta = block.forward(resid, delta, batch, caches[i])
             if observer is not None:
                 # the block's last addend may not be in the stream yet
+                if isinstance(delta, StreamMix):
+                    observer(i + 1, delta.norm_of(ops, resid, None, None, 0.0, torch.float32, store=False))
+                    continue
                 observer(i + 1, resid + delta.float() if isinstance(delta, torch.Tensor) else resid.clone())
         return resid, delta
 
@@ -165,9 +173,14 @@ class DecoderModel:
         The head runs on the wanted rows only (the reference computes all rows of
         a prompt and keeps the last, crates/cuda/src/engine.rs:5685-5720)."""
         resid, delta = self.forward_layers(batch, caches, observer, input_states)
-        if delta is not None and not isinstance(delta, torch.Tensor):
-            delta = None               # a filled norm target: the sum is already in the stream
-        xn = self.final_norm.add_norm(resid, delta, rows=batch.logit_rows)
+        if isinstance(delta, StreamMix):
+            # the model's norm reads the sum of the streams
+            xn = delta.norm_of(kernels.current(), resid, None, self.final_norm.float_weight, self.final_norm.eps, self.dtype,
+                               rows=batch.logit_rows)
+        else:
+            if delta is not None and not isinstance(delta, torch.Tensor):
+                delta = None               # a filled norm target: the sum is already in the stream
+            xn = self.final_norm.add_norm(resid, delta, rows=batch.logit_rows)
         logits = torch.empty((batch.num_logit_rows, self.spec.vocab_size), dtype=torch.float32,
                              device=self.device)
         kernels.current().linear(xn, self.head, logits)

@@ -23,7 +23,10 @@ and ``distance_bias`` (the score is capped by a tanh, and r1_h ln(1 + r2_h (i - 
 its whole size before it is cached, pair m by position * theta^(-2m / size) in the pair layout of the mixer's
 rotation, and a head's result is turned back by the query's position), ``out_gate`` (the concatenated heads times
 sigmoid(W_g h), tensor ``g``) and ``kv_shared`` (no key and value tensors: the layer reads another layer's cache
-with queries of its own). With a head norm and heads that are padded with zeros the norm's mean is taken over
+with queries of its own), ``values_are_keys`` (no value tensor: a value is the key as projected, before its norm and
+rotation; the product makes q and k alone and the head kernel caches k in both places), ``keep_first`` (with a window: a
+request's first tokens stay in sight, and their blocks stay with the request) and ``out_bias`` (a bias on the output
+projection). With a head norm and heads that are padded with zeros the norm's mean is taken over
 the true size: the kernel's mean over D entries with eps * size / D inside the root, times sqrt(size / D) folded
 into the weight, is the same number.
 """
@@ -66,7 +69,7 @@ class GroupedQueryAttention:
     @staticmethod
     def _extended(spec: MixerSpec) -> bool:
         return bool(spec.qk_norm_whole or spec.softcap or spec.distance_bias or spec.rotate_values or spec.out_gate
-                    or spec.kv_shared)
+                    or spec.kv_shared or spec.values_are_keys or spec.keep_first or spec.out_bias)
 
     @classmethod
     def declare_params(cls, spec: MixerSpec, prefix: str) -> List[ParamDecl]:
@@ -77,15 +80,19 @@ class GroupedQueryAttention:
         own_kv = not spec.kv_shared
         out = [ParamDecl(prefix + q, (nq, spec.hidden))]
         if own_kv:
-            out += [ParamDecl(prefix + k, (nkv, spec.hidden)),
-                    ParamDecl(prefix + v, (spec.num_kv_heads * vd, spec.hidden))]
+            out.append(ParamDecl(prefix + k, (nkv, spec.hidden)))
+            if not spec.values_are_keys:
+                out.append(ParamDecl(prefix + v, (spec.num_kv_heads * vd, spec.hidden)))
         out.append(ParamDecl(prefix + o, (spec.hidden, spec.num_heads * vd)))
         if spec.bias:
             bq, bk, bv = cls._bias_names(spec)
             out.append(ParamDecl(prefix + bq, (nq,), init="zeros", role=MATRIX))
             if own_kv:
-                out += [ParamDecl(prefix + bk, (nkv,), init="zeros", role=MATRIX),
-                        ParamDecl(prefix + bv, (spec.num_kv_heads * vd,), init="zeros", role=MATRIX)]
+                out.append(ParamDecl(prefix + bk, (nkv,), init="zeros", role=MATRIX))
+                if not spec.values_are_keys:
+                    out.append(ParamDecl(prefix + bv, (spec.num_kv_heads * vd,), init="zeros", role=MATRIX))
+        if spec.out_bias:
+            out.append(ParamDecl(prefix + o + spec.option("bias_suffix", ".bias"), (spec.hidden,), init="zeros", role=MATRIX))
         if spec.qk_norm or spec.qk_norm_whole:
             nq_name, nk_name = cls._norm_names(spec)
             out.append(ParamDecl(prefix + nq_name, (nq if spec.qk_norm_whole else spec.head_dim,), init="norm", role=VECTOR))
@@ -116,6 +123,11 @@ class GroupedQueryAttention:
         qn, kn, vn, on = self._names(spec)
         H, G = spec.num_heads, spec.num_kv_heads
         self.own_kv = not spec.kv_shared
+        self.values_are_keys = bool(spec.values_are_keys)
+        self.keep = int(spec.keep_first) if self.window else 0
+        if self.values_are_keys and (value_dim != key_dim or spec.kv_shared or spec.qk_norm_whole or spec.rotate_values):
+            raise ValueError("attention: values that are the keys as projected have the keys' size and neither a norm over "
+                             "the whole projection, nor a turn of their own, nor another layer's cache beside them")
         self.extended = self._extended(spec)
         if self.extended:
             # the further options run as kernels of their own around the attention: no norm rides on this
@@ -137,16 +149,23 @@ class GroupedQueryAttention:
         # rows of q, k, v one after the other: stays [out, in], K contiguous
         rows = [heads_of(weights[prefix + qn], H, key_dim)]
         if self.own_kv:
-            rows += [heads_of(weights[prefix + kn], G, key_dim), heads_of(weights[prefix + vn], G, value_dim)]
+            rows.append(heads_of(weights[prefix + kn], G, key_dim))
+            if not self.values_are_keys:
+                rows.append(heads_of(weights[prefix + vn], G, value_dim))
         self.w_qkv = torch.cat(rows, dim=0).contiguous()
         self.b_qkv = None
         if spec.bias:
             bq, bk, bv = self._bias_names(spec)
             rows = [heads_of(weights[prefix + bq], H, key_dim)]
             if self.own_kv:
-                rows += [heads_of(weights[prefix + bk], G, key_dim), heads_of(weights[prefix + bv], G, value_dim)]
+                rows.append(heads_of(weights[prefix + bk], G, key_dim))
+                if not self.values_are_keys:
+                    rows.append(heads_of(weights[prefix + bv], G, value_dim))
             self.b_qkv = torch.cat(rows, dim=0).to(dtype).contiguous()
         self.w_o = weights[prefix + on]
+        self.b_o = None
+        if spec.out_bias:
+            self.b_o = weights[prefix + on + spec.option("bias_suffix", ".bias")].to(dtype).contiguous()
         if value_dim != D:
             wo = torch.zeros((spec.hidden, H, D), dtype=self.w_o.dtype, device=self.w_o.device)
             wo[:, :, :value_dim] = self.w_o.view(spec.hidden, H, value_dim)
@@ -170,6 +189,10 @@ class GroupedQueryAttention:
         self.position = lookup("position", spec.position.kind)(spec.position, device)
         if self.position.rotary_dim > key_dim:
             raise ValueError("the rotated width cannot exceed the head size")
+        # without a rotation the head kernel turns by angles of zero, which changes nothing and takes its fast forms
+        self.rotation = (self.position.inv_freq, self.position.rotary_dim, self.position.style)
+        if self.position.rotary_dim == 0 and self.extended:
+            self.rotation = (torch.zeros(D // 2, dtype=torch.float32, device=device), D, 0)
         self.softcap = float(spec.softcap)
         self.distance = None
         if spec.distance_bias:
@@ -186,7 +209,7 @@ class GroupedQueryAttention:
             self.w_gate = heads_of(weights[prefix + "g"], H, value_dim).contiguous()
 
     def cache_need(self) -> KVNeed:
-        return KVNeed(self.num_kv_heads, self.head_dim, self.window)
+        return KVNeed(self.num_kv_heads, self.head_dim, self.window, self.keep)
 
     def plan_captured_step(self, batch, num_rows: int, ctx_cap: int) -> None:
         # the attention kernels pick their grids by host-side numbers of the step: the kernel set fixes them
@@ -202,7 +225,7 @@ class GroupedQueryAttention:
         # a layer without keys of its own makes queries alone; where the head kernel must still run over them (a
         # head norm, a rotation) the key and value parts it expects are zeros that nothing stores
         head_kernel = self.own_kv or self.q_norm is not None or self.position.rotary_dim > 0
-        width = (H + 2 * G) * D if head_kernel else H * D
+        width = (H + (1 if self.values_are_keys else 2) * G) * D if head_kernel else H * D
         if self.own_kv:
             qkv = torch.empty((T, width), dtype=self.dtype, device=x.device)
             ops.linear(x, self.w_qkv, qkv, self.b_qkv)
@@ -224,11 +247,13 @@ class GroupedQueryAttention:
                            self.value_inv_freq, 1.0)
         slots = batch.slots[cache.group] if (cache.writes and self.own_kv) else batch.no_slots
         if head_kernel:
-            ops.qk_norm_rope_cache(qkv, self.q_norm, self.k_norm, self.eps, batch.positions, self.position.inv_freq,
-                                   self.position.rotary_dim, self.position.style, slots, cache.k, cache.v, H, G, D)
+            inv_freq, rotary_dim, style = self.rotation
+            more = {"values_are_keys": True} if self.values_are_keys else {}
+            ops.qk_norm_rope_cache(qkv, self.q_norm, self.k_norm, self.eps, batch.positions, inv_freq, rotary_dim, style,
+                                   slots, cache.k, cache.v, H, G, D, **more)
         attn = torch.empty((T, H * D), dtype=self.dtype, device=x.device)
         ops.attention(qkv, width, attn, cache.k, cache.v, batch, H, G, D, self.scale, self.window, cache.group,
-                      softcap=self.softcap, distance=self.distance)
+                      softcap=self.softcap, distance=self.distance, **({"keep": self.keep} if self.keep else {}))
         if self.value_inv_freq is not None or self.w_gate is not None:
             gate = None
             if self.w_gate is not None:
@@ -238,7 +263,7 @@ class GroupedQueryAttention:
             ops.turn_heads(attn, H, D, turned, self.position.style, batch.positions, self.value_inv_freq, -1.0,
                            gate=gate, gate_stride=D)
         out = torch.empty((T, self.spec.hidden), dtype=torch.float32, device=x.device)
-        ops.linear(attn, self.w_o, out)
+        ops.linear(attn, self.w_o, out, self.b_o)
         return out
 
     def forward(self, x, batch, cache: LayerCache, resid: Optional[torch.Tensor] = None,

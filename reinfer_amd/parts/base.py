@@ -15,9 +15,10 @@ class PagedNeed:
     engine allocates ``[blocks, *shape]`` for each and hands them over in ``LayerCache.tensors`` by name;
     token slot s of the step (``batch.slots[group]``) is slot ``s % block_size`` of block ``s // block_size``,
     wherever in its block's shape the mixer puts it. ``window`` W > 0: only the last W tokens are read, the
-    blocks behind them go back to the pool."""
+    blocks behind them go back to the pool, but for those that hold the request's first ``keep`` tokens."""
     tensors: Tuple[Tuple[str, Tuple[int, ...], Optional[torch.dtype]], ...]
     window: int = 0
+    keep: int = 0
 
     def block_tensors(self, block_size: int):
         return tuple((name, tuple(block_size if n == -1 else n for n in shape), dtype)
@@ -26,12 +27,13 @@ class PagedNeed:
 
 @dataclass(frozen=True)
 class KVNeed:
-    """Keys and values of every token (``window`` 0) or of the last ``window`` tokens, as the attention
-    kernels read them: tensors "k" and "v", a block of each ``[kv_heads, block_size // 16, 16 * head_dim]``,
+    """Keys and values of every token (``window`` 0) or of the last ``window`` tokens (and of a request's first
+    ``keep`` tokens), as the attention kernels read them: tensors "k" and "v", a block of each ``[kv_heads, block_size // 16, 16 * head_dim]``,
     tiles of 16 slots in matrix-core operand order (:mod:`reinfer_amd.cache.layout`)."""
     num_kv_heads: int
     head_dim: int
     window: int = 0
+    keep: int = 0           # first tokens that a window keeps in sight
 
     def block_tensors(self, block_size: int):
         from ..cache.layout import cache_shape
@@ -144,6 +146,31 @@ class StreamCopy:
     holds the stream in the activations' type (``x`` [T, width]): a block whose parts read the stream itself takes
     it as their operand; any other block treats it as "nothing pending"."""
     x: torch.Tensor
+
+
+@dataclass
+class StreamMix:
+    """What a block of several residual streams hands on: a sublayer's result ``y`` that is not in the streams yet, with
+    the sublayer's ``mix`` [from, to] and ``w_out``, X_t <- sum_s mix[s, t] X_s + w_out[t] y; ``base`` [T, width]: every
+    stream is still this row (the model's start), the streams' own buffer holds nothing yet."""
+    base: Optional[torch.Tensor] = None
+    y: Optional[torch.Tensor] = None
+    mix: Optional[torch.Tensor] = None
+    w_out: Optional[torch.Tensor] = None
+
+    def norm_of(self, ops, streams: torch.Tensor, w_in: Optional[torch.Tensor], weight: Optional[torch.Tensor], eps: float,
+                dtype: torch.dtype, rows: Optional[torch.Tensor] = None, store: bool = True) -> torch.Tensor:
+        """The norm of the weighted sum of the streams (``w_in`` None: their sum; ``weight`` None: no norm) after what is
+        pending; the new streams are kept where there was something pending, unless ``rows`` asks for some rows alone."""
+        T, _, width = streams.shape
+        out = torch.empty((T if rows is None else rows.numel(), width), dtype=dtype, device=streams.device)
+        ops.hyper_step(streams, self.base, self.y, self.mix, self.w_out, w_in, weight, eps, out, rows=rows,
+                       store=store and rows is None and self.y is not None)
+        return out
+
+    def stored(self) -> "StreamMix":
+        """What is left pending once :meth:`norm_of` has kept the new streams."""
+        return self if self.y is None else StreamMix()
 
 
 @dataclass

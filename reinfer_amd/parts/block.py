@@ -54,6 +54,7 @@ class PreNormBlock:
                                                                p + spec.ffn_norm_name, dtype, device)
             self.ffn = lookup("feed_forward", spec.ffn.kind)(spec.ffn, weights, p + spec.ffn_prefix, dtype, device)
         self.residual_scale = float(spec.residual_scale)
+        self.dtype = dtype
         # the norm-on-products hand-over is for the plain form: both parts there, addends entering as they are
         self.passes_emit = self.ffn is not None and self.residual_scale == 1.0
 
@@ -95,7 +96,7 @@ class PreNormBlock:
             else:
                 a = mixer.forward(xn, batch, cache, resid=resid)
         else:
-            a = mixer.forward(xn, batch, cache)
+            a = self._same_dtype(mixer.forward(xn, batch, cache), resid)
         xn = self._norm(self.ffn_norm, resid, a, ffn)
         if getattr(ffn, "adds_in_place", False):
             if emit is not None and getattr(ffn, "emits_for_norm", False):
@@ -115,12 +116,23 @@ class PreNormBlock:
             delta = None               # a filled norm target: the sum is already in the stream
         xn = self.mixer_norm.add_norm(resid, delta)
         a = self._run(self.mixer, xn, batch, resid, s, cache)
+        if s == 1.0:
+            a = self._same_dtype(a, resid)
         if self.ffn is not None:
             xn = self.ffn_norm.add_norm(resid, a, delta_scale=s) if a is not None else self.ffn_norm.add_norm(resid, None)
             a = self._run(self.ffn, xn, batch, resid, s)
         if a is not None:
             kernels.current().stream_add(resid, a, delta_scale=s)
         return None
+
+    def _same_dtype(self, a, resid):
+        """An addend for the norm behind it, which takes it in the activations' type; a result of another type goes into
+        the stream by itself."""
+        if isinstance(a, torch.Tensor) and a.dtype != self.dtype:
+            from .. import kernels
+            kernels.current().stream_add(resid, a)
+            return None
+        return a
 
     @staticmethod
     def _run(part, xn, batch, resid, s, *cache):

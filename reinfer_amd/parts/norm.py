@@ -41,7 +41,19 @@ class RMSNorm:
         if spec.offset:
             # a weight stored around zero: the factor offset + w is made once, in float
             self.weight = (weights[name].float() + float(spec.offset)).contiguous()
+        if float(getattr(spec, "factor", 1.0)) != 1.0:
+            # a constant behind a linear map of the norm: made part of the weight once, in float
+            self.weight = (self.weight.float() * float(spec.factor)).contiguous()
         self.dtype = dtype
+
+    @property
+    def float_weight(self) -> torch.Tensor:
+        """The weight as float32, for kernels that take no other."""
+        if self.weight.dtype != torch.float32:
+            if getattr(self, "_float_weight", None) is None:
+                self._float_weight = self.weight.float().contiguous()
+            return self._float_weight
+        return self.weight
 
     def add_norm(self, resid: torch.Tensor, delta, rows: Optional[torch.Tensor] = None,
                  scaled_ok: bool = False, delta_scale: float = 1.0):

@@ -45,11 +45,12 @@ class KernelDouble:
         out.copy_(((xg * rstd).reshape(n, h) * weight.float()).to(out.dtype))
 
     def qk_norm_rope_cache(self, qkv, q_weight, k_weight, eps, positions, inv_freq, rotary_dim,
-                           rope_style, slots, kcache, vcache, num_heads, num_kv_heads, head_dim):
+                           rope_style, slots, kcache, vcache, num_heads, num_kv_heads, head_dim, values_are_keys=False):
         T = qkv.shape[0]
         d = head_dim
-        u = qkv.view(T, num_heads + 2 * num_kv_heads, d).float()
-        q, k, v = u[:, :num_heads], u[:, num_heads:num_heads + num_kv_heads], u[:, num_heads + num_kv_heads:]
+        u = qkv.view(T, num_heads + (1 if values_are_keys else 2) * num_kv_heads, d).float()
+        q, k = u[:, :num_heads], u[:, num_heads:num_heads + num_kv_heads]
+        v = k if values_are_keys else u[:, num_heads + num_kv_heads:]
 
         def norm(x, w):
             if w is None:
@@ -205,7 +206,8 @@ class KernelDouble:
         T = read.shape[0]
         o = read.view(T, H, dv)
         o = o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps)
-        o = o * (weight.view(H, dv) if per_head else weight.view(1, dv))
+        if weight is not None:
+            o = o * (weight.view(H, dv) if per_head else weight.view(1, dv))
         g = gate[:, :H * dv].float().view(T, H, dv)
         g = torch.sigmoid(g) if kind == "sigmoid" else g * torch.sigmoid(g)
         out.copy_((o * g).reshape(T, H * dv).to(out.dtype))
@@ -269,9 +271,20 @@ class KernelDouble:
                 out[t] = torch.einsum("hkv,hk->hv", S + uu[:, :, None] * kv, r).reshape(-1)
                 S.mul_(w[t][:, :, None]).add_(kv)
 
-    def decay_scan(self, proj, q_off, k_off, v_off, decays, state, batch, H, dk, dv, out):
-        p = proj.float()
-        p = p * torch.sigmoid(p)
+    def decay_scan(self, proj, q_off, k_off, v_off, decays, state, batch, H, dk, dv, out, act="silu", inv_freq=None,
+                   rot_dims=0, q_scale=1.0, k_scale=1.0):
+        p = proj.float().clone()
+        if act == "silu":
+            p = p * torch.sigmoid(p)
+        half = rot_dims // 2
+        for off, scale in ((q_off, q_scale), (k_off, k_scale)):
+            x = p[:, off:off + H * dk].view(-1, H, dk)
+            if half:
+                ang = batch.positions.float()[:, None] * inv_freq[:half][None, :]
+                c, s = torch.cos(ang)[:, None], torch.sin(ang)[:, None]
+                a, b = x[..., :half].clone(), x[..., half:rot_dims].clone()
+                x[..., :half], x[..., half:rot_dims] = a * c - b * s, b * c + a * s
+            x *= scale
         for first, rows, slot, fresh in self._requests(batch):
             if slot < 0:
                 out[first:first + rows] = 0
@@ -285,6 +298,38 @@ class KernelDouble:
                 v = p[t, v_off:v_off + H * dv].view(H, dv)
                 S.mul_(decays.float()[:, None, None]).add_(k[:, :, None] * v[:, None, :])
                 out[t] = torch.einsum("hkv,hk->hv", S, q).reshape(-1)
+
+    def gated_linear_scan(self, proj, q_off, k_off, v_off, z, bias, tau, state, batch, H, dk, dv, out, q_scale=1.0):
+        p = proj.float()
+        alpha = torch.exp(torch.nn.functional.logsigmoid(z[:, :H * dk] + bias) / tau).view(-1, H, dk)
+        for first, rows, slot, fresh in self._requests(batch):
+            if slot < 0:
+                out[first:first + rows] = 0
+                continue
+            S = state[slot, :H * dk * dv].view(H, dk, dv)
+            if fresh:
+                S.zero_()
+            for t in range(first, first + rows):
+                q = p[t, q_off:q_off + H * dk].view(H, dk) * q_scale
+                k = p[t, k_off:k_off + H * dk].view(H, dk)
+                v = p[t, v_off:v_off + H * dv].view(H, dv)
+                S.mul_(alpha[t][:, :, None]).add_(k[:, :, None] * v[:, None, :])
+                out[t] = torch.einsum("hkv,hk->hv", S, q).reshape(-1)
+
+    # ---- several residual streams
+    def hyper_step(self, streams, base, y, mix, w_out, w_in, weight, eps, out, rows=None, store=True):
+        X = streams if base is None else base[:, None, :].expand_as(streams)
+        if y is not None:
+            X = torch.einsum("st,nsw->ntw", mix, X) + w_out[None, :, None] * y.float()[:, None, :]
+        if rows is not None:
+            X = X[rows.long()]
+        elif store:
+            streams.copy_(X)
+        u = X.sum(1) if w_in is None else (X * w_in[None, :, None]).sum(1)
+        if weight is not None:
+            u = u * torch.rsqrt((u * u).mean(-1, keepdim=True) + eps) * weight
+        if out is not None:
+            out.copy_(u.to(out.dtype))
 
     # ---- sublayers that read the stream, results behind a norm
     def stream_cast(self, resid, out):
@@ -549,7 +594,7 @@ class KernelDouble:
                 so[p] = sq[:, p * part:(p + 1) * part].sum(1)
 
     def attention(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
-                  scale, window, group, softcap=0.0, distance=None):
+                  scale, window, group, softcap=0.0, distance=None, keep=0):
         T = batch.num_tokens
         bs = kcache.shape[2] * 16
         kl, vl = unpack_k(kcache, head_dim), unpack_v(vcache, head_dim)      # [blocks, Hkv, bs, d]
@@ -560,7 +605,7 @@ class KernelDouble:
             seq = int(batch.seq_of_token[t])
             p = int(batch.positions[t])
             lo = max(0, p - window + 1) if window > 0 else 0
-            keys = torch.arange(lo, p + 1)
+            keys = torch.cat([torch.arange(0, min(keep, lo)), torch.arange(lo, p + 1)])
             blk = tables[seq, keys // bs].long()
             K = kl[blk, :, keys % bs, :].float()        # [n, Hkv, d]
             V = vl[blk, :, keys % bs, :].float()
