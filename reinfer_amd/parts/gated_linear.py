@@ -44,11 +44,13 @@ class GatedLinear:
         self.heads, self.key_dim, self.value_dim, self.rank = int(p.heads), int(p.key_dim), int(p.value_dim), int(p.rank)
         self.tau, self.q_scale, self.norm_eps = float(p.tau), float(p.q_scale), float(p.norm_eps)
         self.width = int(spec.hidden)
-        parts = [weights[prefix + s] for s in ("q", "k", "v", "g", "a1")]
-        # the low-rank input is read out of the product's rows by the next product: the rows end on a multiple of 8
-        pad = -sum(w.shape[0] for w in parts) % 8
-        if pad:
-            parts.append(torch.zeros((pad, self.width), dtype=parts[0].dtype, device=parts[0].device))
+        # the next product reads the low-rank input out of this product's rows: it starts and the rows end on a multiple
+        # of 8 (16 bytes), with rows of zeros before and behind it where the sizes want them
+        parts = [weights[prefix + s] for s in ("q", "k", "v", "g")]
+        rows = 2 * self.heads * (self.key_dim + self.value_dim)
+        self.low_at = -(-rows // 8) * 8
+        zeros = lambda n: torch.zeros((n, self.width), dtype=parts[0].dtype, device=parts[0].device)
+        parts += [zeros(self.low_at - rows), weights[prefix + "a1"], zeros(-self.rank % 8)]
         self.w_in = torch.cat(parts, dim=0).contiguous()
         self.w_a2 = weights[prefix + "a2"]
         self.b_a2 = weights[prefix + "a2.b"].float().contiguous()
@@ -64,19 +66,15 @@ class GatedLinear:
         ops = kernels.current()
         T = x.shape[0]
         nk, nv = self.heads * self.key_dim, self.heads * self.value_dim
-        low_at = 2 * nk + 2 * nv
         proj = torch.empty((T, self.w_in.shape[0]), dtype=self.dtype, device=x.device)
         ops.linear(x, self.w_in, proj)
-        low = proj[:, low_at:low_at + self.rank]
-        if low_at % 8 or self.rank % 8:
-            low = low.contiguous()              # a product's rows start on 16 bytes
         z = torch.empty((T, nk), dtype=torch.float32, device=x.device)      # pre-activation, kept in float
-        ops.linear(low, self.w_a2, z)
+        ops.linear(proj[:, self.low_at:self.low_at + self.rank], self.w_a2, z)
         read = torch.empty((T, nv), dtype=torch.float32, device=x.device)
         ops.gated_linear_scan(proj, 0, nk, 2 * nk, z, self.b_a2, self.tau, cache.state, batch, self.heads, self.key_dim,
                               self.value_dim, read, q_scale=self.q_scale)
         act = torch.empty((T, nv), dtype=self.dtype, device=x.device)
-        ops.head_norm_gate(read, self.norm_weight, False, proj[:, 2 * nk + nv:low_at], "silu", self.norm_eps, self.heads,
+        ops.head_norm_gate(read, self.norm_weight, False, proj[:, 2 * nk + nv:2 * nk + 2 * nv], "silu", self.norm_eps, self.heads,
                            self.value_dim, act)
         out = torch.empty((T, self.width), dtype=torch.float32, device=x.device)     # enters a float sum as it is
         ops.linear(act, self.w_o, out)

@@ -45,11 +45,11 @@ def turn_halves(x: torch.Tensor, pos: torch.Tensor, n: int, base: float) -> torc
 
 
 # ------------------------------------------------------------------ linear attention with a fixed decay a head
-def retention(h, w, p, cfg, eps):
+def retention(h, w, p, cfg, eps, noise=lambda x: x):
     H, dk, dv = cfg["heads"], cfg["dim"], cfg["vdim"]
     T = h.shape[0]
-    q, k = (h @ w[p + "q"].T).view(T, H, dk), (h @ w[p + "k"].T).view(T, H, dk)
-    v = (h @ w[p + "v"].T).view(T, H, dv)
+    q, k = noise(h @ w[p + "q"].T).view(T, H, dk), noise(h @ w[p + "k"].T).view(T, H, dk)
+    v = noise(h @ w[p + "v"].T).view(T, H, dv)
     rot = cfg.get("rot")
     if rot:
         pos = torch.arange(T)
@@ -70,11 +70,11 @@ def visible(i: int, j: int, window: int, first: int) -> bool:
     return j <= i and (window == 0 or i - j < window or j < first)
 
 
-def sink_attention(h, w, p, cfg, eps):
+def sink_attention(h, w, p, cfg, eps, noise=lambda x: x):
     H, G, d = cfg["heads"], cfg["kv_heads"], cfg["dim"]
     T = h.shape[0]
-    q = (h @ w[p + "q"].T + w[p + "q.b"]).view(T, H, d)
-    raw = (h @ w[p + "k"].T + w[p + "k.b"]).view(T, G, d)
+    q = noise(h @ w[p + "q"].T + w[p + "q.b"]).view(T, H, d)
+    raw = noise(h @ w[p + "k"].T + w[p + "k.b"]).view(T, G, d)
     v = raw                                                    # the keys before their norm
     q = rms(q, eps) * w[p + "q.norm"]
     k = rms(raw, eps) * w[p + "k.norm"]
@@ -91,12 +91,12 @@ def sink_attention(h, w, p, cfg, eps):
 
 
 # ------------------------------------------------------------------ linear attention with a gated decay a key channel
-def gla(h, w, p, cfg, eps):
+def gla(h, w, p, cfg, eps, noise=lambda x: x):
     H, dk, dv = cfg["heads"], cfg["dim"], cfg["vdim"]
     T = h.shape[0]
-    q = (h @ w[p + "q"].T).view(T, H, dk) * dk ** -0.5
-    k = (h @ w[p + "k"].T).view(T, H, dk)
-    v = (h @ w[p + "v"].T).view(T, H, dv)
+    q = noise(h @ w[p + "q"].T).view(T, H, dk) * dk ** -0.5
+    k = noise(h @ w[p + "k"].T).view(T, H, dk)
+    v = noise(h @ w[p + "v"].T).view(T, H, dv)
     z = (h @ w[p + "a1"].T) @ w[p + "a2"].T + w[p + "a2.b"]
     alpha = (torch.sigmoid(z) ** (1.0 / cfg["tau"])).view(T, H, dk)
     out = torch.zeros(T, H, dv, dtype=D)
@@ -137,9 +137,12 @@ def run_order(raw: dict) -> List[int]:
     return list(range(a)) + list(range(a, b)) * k + list(range(b, n))
 
 
-def forward(raw: dict, w: Dict[str, torch.Tensor], tokens: Sequence[int], layers_out: Optional[list] = None):
+def forward(raw: dict, w: Dict[str, torch.Tensor], tokens: Sequence[int], layers_out: Optional[list] = None,
+            noise=None):
     """Logits [T, vocab] of one sequence from its start; ``layers_out`` collects the sum of the streams behind every
-    layer run."""
+    layer run. ``noise`` (a function of a tensor) is put on what every sublayer reads and returns and on a mixer's
+    queries, keys and values: how far that moves the logits is how far roundings of its size may."""
+    noise = noise or (lambda x: x)
     w = {k: t.to(D) for k, t in w.items()}
     eps = float(raw["norm"]["eps"])
     x = w["embed"][torch.tensor(list(tokens))] * float((raw.get("embedding") or {}).get("scale", 1.0))
@@ -149,14 +152,14 @@ def forward(raw: dict, w: Dict[str, torch.Tensor], tokens: Sequence[int], layers
     def sublayer(X, p, q, part):
         if n is None:
             u = X[0]
-            return (u + part(rms(u, eps) * w[f"{p}norm{q}"]))[None]
+            return (u + noise(part(noise(rms(u, eps) * w[f"{p}norm{q}"]))))[None]
         c = f"{p}hc{q}."
-        y = part(rms(combine(X, w[c + "in"]), eps) * w[f"{p}norm{q}"])
+        y = noise(part(noise(rms(combine(X, w[c + "in"]), eps) * w[f"{p}norm{q}"])))
         return spread(X, y, w[c + "mix"], w[c + "out"])
 
     for i in run_order(raw):
         L, p = raw["layers"][i], f"l{i}."
-        X = sublayer(X, p, 1, lambda h: MIXERS[L["type"]](h, w, p + "mix.", L["mixer"], eps))
+        X = sublayer(X, p, 1, lambda h: MIXERS[L["type"]](h, w, p + "mix.", L["mixer"], eps, noise))
         if L.get("mlp") is not None:
             X = sublayer(X, p, 2, lambda h: swiglu(h, w, p + "mlp."))
         if layers_out is not None:

@@ -46,6 +46,40 @@ def test_plan_groups():
     assert [(g.window, g.entries) for g in groups] == [(0, (0, 3)), (4, (5,)), (8, (1, 4))]
 
 
+def test_plan_groups_tells_windows_that_keep_first_tokens_apart():
+    groups = plan_groups([8, 8, None, 0, 8, 4], [0, 3, 0, 5, 3, 0])
+    assert [(g.window, g.keep, g.entries) for g in groups] == [(0, 0, (3,)), (4, 0, (5,)), (8, 0, (0,)), (8, 3, (1, 4))]
+
+
+def test_a_window_keeps_the_blocks_of_its_first_tokens():
+    """Blocks of four tokens, a window of six, five kept tokens: the first two blocks stay with the request, the blocks
+    between them and the window go back, and all come back once at the end."""
+    m = CacheManager([CacheGroupSpec(window=6, entries=(0,), keep=5)], 4, [8], 2)
+    m.add("a")
+    held = []
+    for total in range(1, 41):
+        m.grow("a", total)
+        m.commit("a", total)
+        m.check()
+        table = m.get("a").tables[0]
+        live = [b for b, x in enumerate(table) if x >= 0]
+        first = max(0, total - 6 + 1) // 4
+        assert live == sorted({b for b in range(len(table)) if b < 2 or b >= first}), (total, live)
+        held.append(len(live))
+    assert max(held) <= 5 and m.slot_of("a", 0, 4) >= 0 and m.slot_of("a", 0, 12) == -1
+    assert m.blocks_needed("a", 41) == [1]
+    # a whole prompt in one step takes all of its blocks, and gives back those in between behind it
+    m.add("b")
+    assert m.blocks_needed("b", 16) == [4]
+    m.free("a")
+    m.grow("b", 30)
+    m.commit("b", 30)
+    assert [x >= 0 for x in m.get("b").tables[0]] == [True, True, False, False, False, False, True, True]
+    m.free("b")
+    m.check()
+    assert m.pools[0].num_free == 8
+
+
 def manager(num_blocks=8, windows=(0,), bs=4, max_seqs=4):
     groups = [CacheGroupSpec(window=w, entries=(i,)) for i, w in enumerate(windows)]
     return CacheManager(groups, bs, [num_blocks] * len(groups), max_seqs)
