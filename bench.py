@@ -540,6 +540,47 @@ def gibavik_sizes():
     return out
 
 
+# ---------------------------------------------------------------------------------------------------
+# --design sagalorn: the Sagalorn design beside the Gibavik design (the closest of the others: attention inside a window
+# with biases and head norms, a memory that fades by a constant, a dense feed-forward) at equal size
+# ---------------------------------------------------------------------------------------------------
+def _sagalorn_raw(width, vocab, pattern, attn, heads, ff):
+    """``pattern``: a string of layer codes, R retention, A attention, G gated linear attention, each with a dense
+    feed-forward."""
+    H, kv = attn
+    mixers = {"R": ("retention", {"decay": [1.0 - 2.0 ** -(4 + 6 * h / max(1, heads - 1)) for h in range(heads)], "dim": 128,
+                                  "heads": heads, "rot": {"base": 10000.0, "dims": 128}, "vdim": 128}),
+              "A": ("attention", {"dim": 128, "heads": H, "kv_heads": kv, "mask": {"keep_first": 4, "size": 1024},
+                                  "scale": 128 ** -0.5, "vdim": 128}),
+              "G": ("gla", {"dim": 64, "heads": heads, "tau": 16.0, "vdim": 128})}
+    return {"architecture": "Sagalorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 6.0},
+            "logit_scale": 0.5, "streams": 4, "gla_ranks": [16 if c == "G" else 0 for c in pattern],
+            "layers": [{"type": mixers[c][0], "mixer": mixers[c][1], "mlp": {"ff": ff, "kind": "dense"}} for c in pattern]}
+
+
+# (name, Sagalorn configuration, its Gibavik twin, vocabulary, "gibavik"): as many layers, the same width and heads; an
+# attention layer for an attention layer (window 1,024 both) and a side-by-side layer (attention + memory) for a layer of
+# linear attention (Gibavik has none of a memory alone); the twin's feed-forward width (a multiple of 64) brings its
+# parameter count closest to Sagalorn's
+def sagalorn_sizes():
+    out = []
+    for name, width, attn, heads, ff in (("w2048", 2048, (16, 4), 16, 5632), ("w4096", 4096, (32, 8), 32, 11008)):
+        vocab, pattern = 32768, "RAGRAG"
+        raw = _sagalorn_raw(width, vocab, pattern, attn, heads, ff)
+
+        def twin(tff):
+            g = _gibavik_raw(width, vocab, "".join("A" if c == "A" else "p" for c in pattern), attn, heads, tff, (1, 1, 64))
+            for L in g["layers"]:
+                L["mlp"] = {"ff": tff, "kind": "dense", "limit": 7.0}
+                if L["type"] == "attention":
+                    L["mixer"] = dict(L["mixer"], mask={"size": 1024})
+            return g
+        want, a, b = _parameters(raw), _parameters(twin(1024)), _parameters(twin(2048))
+        tff = max(64, round((1024 + (want - a) * 1024 / (b - a)) / 64) * 64)
+        out.append((name, raw, twin(tff), vocab, "gibavik"))
+    return out
+
+
 def design_run(args) -> int:
     """Prefill and decode throughput of the design (``--design``) and of its twin at each size, and the GPU time of a
     2,048-token prompt step and of a decode step at batch 8 by kernel class with each class's share of its
@@ -583,7 +624,7 @@ def design_run(args) -> int:
 
     results = {}
     sizes = {"kobolix": kobolix_sizes, "puresun": design_sizes, "detatar": detatar_sizes,
-             "gibavik": gibavik_sizes}[args.design]()
+             "gibavik": gibavik_sizes, "sagalorn": sagalorn_sizes}[args.design]()
     twin_name = "qwen3"
     for name, p_raw, q_raw, vocab, *rest in sizes:
         twin_name = rest[0] if rest else "qwen3"
@@ -642,9 +683,9 @@ def main() -> int:
     ap.add_argument("--max-model-len", type=int, default=None, metavar="N",
                     help="context length (default: the shape's: 4096 at 8b, 8192 at 4b, 16384 at 32b)")
     ap.add_argument("--shape", default="8b", choices=sorted(SHAPES), help="layer sizes (default: the Qwen3-8B shape)")
-    ap.add_argument("--design", default=None, choices=["puresun", "kobolix", "detatar", "gibavik"],
+    ap.add_argument("--design", default=None, choices=["puresun", "kobolix", "detatar", "gibavik", "sagalorn"],
                     help="instead of the default measurement: this design beside its closest other (the Qwen3 decoder; "
-                         "for detatar, Puresun) at equal sizes")
+                         "for detatar, Puresun; for gibavik, Kobolix; for sagalorn, Gibavik) at equal sizes")
     ap.add_argument("--size", default=None, help="with --design: this size alone (w2048 or w4096)")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -168,7 +168,7 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p) {
             const float pk = to_f32(kg[row0 + kq_g[j] + o]) * p.k_scale;
             const float pq = to_f32(qg[row0 + kq_g[j] + o]) * p.q_scale;
             float sn, cs;
-            sincosf((float)p.positions[t0 + kq_t[j]] * p.inv_freq[lower ? e : e - half], &sn, &cs);
+            ra_sincos((float)p.positions[t0 + kq_t[j]] * p.inv_freq[lower ? e : e - half], &sn, &cs);
             if (lower) sn = -sn;
             fk[j] = fk[j] * cs + pk * sn;
             fq[j] = fq[j] * cs + pq * sn;

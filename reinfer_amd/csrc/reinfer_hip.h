@@ -325,15 +325,17 @@ int ra_gla_scan(const void* proj, int act_dtype, int ld, int q_off, int k_off, i
                 const int* state_slots, const int* fresh, int n_seqs, int n_tokens, int max_q_len, int heads, int key_dim,
                 int value_dim, float* out, hipStream_t stream);
 // The same recurrences (silu: ra_decay_scan's) in chunks of 16 tokens on the float matrix cores, keys up to 256, from and
-// into the same state. Scratch: turn n_tokens * rot_dims floats; cum n_tokens * heads * key_dim floats.
+// into the same state. Scratch: ra_chunk_scratch_floats(...) floats, 16-byte aligned.
+long ra_chunk_scratch_floats(int n_tokens, int n_seqs, int heads, int key_dim, int value_dim);
 int ra_decay_chunks(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off, int silu, const float* decays,
-                    const int* positions, const float* inv_freq, int rot_dims, float* turn, float q_scale, float k_scale,
-                    float* state, long slot_stride, const int* cu_tokens, const int* state_slots, const int* fresh,
-                    int n_seqs, int n_tokens, int heads, int key_dim, int value_dim, float* out, hipStream_t stream);
+                    const int* positions, const float* inv_freq, int rot_dims, float q_scale, float k_scale, float* state,
+                    long slot_stride, const int* cu_tokens, const int* state_slots, const int* fresh, int n_seqs,
+                    int n_tokens, int heads, int key_dim, int value_dim, float* scratch, long scratch_floats, float* out,
+                    hipStream_t stream);
 int ra_gla_chunks(const void* proj, int act_dtype, int ld, int q_off, int k_off, int v_off, const float* z, int ldz,
-                  const float* bias, float tau, float* cum, float q_scale, float* state, long slot_stride,
-                  const int* cu_tokens, const int* state_slots, const int* fresh, int n_seqs, int n_tokens, int max_q_len,
-                  int heads, int key_dim, int value_dim, float* out, hipStream_t stream);
+                  const float* bias, float tau, float q_scale, float* state, long slot_stride, const int* cu_tokens,
+                  const int* state_slots, const int* fresh, int n_seqs, int n_tokens, int heads, int key_dim, int value_dim,
+                  float* scratch, long scratch_floats, float* out, hipStream_t stream);
 // Several residual streams: X_t <- sum_s mix[s, t] X_s + w_out[t] y (y null: as they are; base: every stream is this row),
 // u = sum_t w_in[t] X_t (null: ones); out = u / sqrt(mean u^2 + eps) * weight (weight null: u). store: keep the new streams.
 int ra_hyper_step(float* streams, const float* base, const void* y, int y_dtype, const float* mix, const float* w_out,

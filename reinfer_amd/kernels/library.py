@@ -85,8 +85,8 @@ _SIGNATURES = {
     "ra_decay_scan": [P, I, I, I, I, I, P, P, c_long, P, P, P, I, I, I, I, I, I, P, P],
     "ra_retention_scan": [P, I, I, I, I, I, P, P, P, I, F, F, P, c_long, P, P, P, I, I, I, I, I, I, P, P],
     "ra_gla_scan": [P, I, I, I, I, I, P, I, P, F, F, P, c_long, P, P, P, I, I, I, I, I, I, P, P],
-    "ra_decay_chunks": [P, I, I, I, I, I, I, P, P, P, I, P, F, F, P, c_long, P, P, P, I, I, I, I, I, P, P],
-    "ra_gla_chunks": [P, I, I, I, I, I, P, I, P, F, P, F, P, c_long, P, P, P, I, I, I, I, I, I, P, P],
+    "ra_decay_chunks": [P, I, I, I, I, I, I, P, P, P, I, F, F, P, c_long, P, P, P, I, I, I, I, I, P, c_long, P, P],
+    "ra_gla_chunks": [P, I, I, I, I, I, P, I, P, F, F, P, c_long, P, P, P, I, I, I, I, I, P, c_long, P, P],
     "ra_hyper_step": [P, P, P, I, P, P, P, P, F, P, I, I, I, I, P, I, P],
     "ra_moe_table_route": [P, P, I, P, P, I, P],
     "ra_stream_cast": [P, P, I, c_long, P],
@@ -132,6 +132,8 @@ def load() -> ctypes.CDLL:
         lib.ra_sample_static_max_pairs.argtypes = []
         lib.ra_sample_static_prepare.restype = c_int
         lib.ra_sample_static_prepare.argtypes = []
+        lib.ra_chunk_scratch_floats.restype = c_long
+        lib.ra_chunk_scratch_floats.argtypes = [c_int, c_int, c_int, c_int, c_int]
         lib.ra_scan_state_floats.restype = c_long
         lib.ra_scan_state_floats.argtypes = [c_int, c_int, c_int, c_int]
         lib.ra_gemm_skinny_max_rows.restype = c_int

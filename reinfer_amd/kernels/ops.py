@@ -1333,6 +1333,13 @@ class HipKernels:
         if out.shape != (T, heads * value_dim) or out.dtype != torch.float32 or not out.is_contiguous():
             raise ValueError(f"{what}: out is contiguous float32 [T, {heads * value_dim}]")
 
+    @staticmethod
+    def _chunk_scratch(T, n_seqs, heads, key_dim, value_dim, device) -> torch.Tensor:
+        n = int(library.load().ra_chunk_scratch_floats(T, n_seqs, int(heads), int(key_dim), int(value_dim)))
+        if n < 0:
+            raise ValueError(f"heads of {key_dim} x {value_dim} are not taken in chunks (keys up to 256)")
+        return torch.empty(n, dtype=torch.float32, device=device)
+
     def decay_scan(self, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, decays: torch.Tensor,
                    state: torch.Tensor, batch, heads: int, key_dim: int, value_dim: int, out: torch.Tensor,
                    act: str = "silu", inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0,
@@ -1365,10 +1372,11 @@ class HipKernels:
                 batch.fresh.data_ptr(), batch.num_seqs, T)
         turned = (batch.positions.data_ptr() if rot_dims else None, _ptr(inv_freq) if rot_dims else None, int(rot_dims))
         if chunks:
-            turn = torch.empty(T * rot_dims, dtype=torch.float32, device=proj.device) if rot_dims else None
+            scratch = self._chunk_scratch(T, batch.num_seqs, heads, key_dim, value_dim, proj.device)
             library.call("ra_decay_chunks", proj.data_ptr(), tag, proj.stride(0), int(q_off), int(k_off), int(v_off),
-                         1 if act == "silu" else 0, decays.data_ptr(), *turned, _ptr(turn), float(q_scale), float(k_scale),
-                         *tail, int(heads), int(key_dim), int(value_dim), out.data_ptr(), _stream())
+                         1 if act == "silu" else 0, decays.data_ptr(), *turned, float(q_scale), float(k_scale), *tail,
+                         int(heads), int(key_dim), int(value_dim), scratch.data_ptr(), scratch.numel(), out.data_ptr(),
+                         _stream())
         elif act == "silu":
             library.call("ra_decay_scan", proj.data_ptr(), tag, proj.stride(0), int(q_off), int(k_off), int(v_off),
                          decays.data_ptr(), *tail, longest, int(heads), int(key_dim), int(value_dim), out.data_ptr(),
@@ -1399,13 +1407,13 @@ class HipKernels:
         head = (proj.data_ptr(), tag, proj.stride(0), int(q_off), int(k_off), int(v_off), z.data_ptr(), z.stride(0),
                 bias.data_ptr(), float(tau))
         tail = (float(q_scale), state.data_ptr(), state.stride(0), batch.cu_tokens.data_ptr(),
-                batch.state_slots.data_ptr(), batch.fresh.data_ptr(), batch.num_seqs, T, longest, int(heads), int(key_dim),
-                int(value_dim), out.data_ptr(), _stream())
+                batch.state_slots.data_ptr(), batch.fresh.data_ptr(), batch.num_seqs, T)
+        sizes = (int(heads), int(key_dim), int(value_dim))
         if chunks:
-            cum = torch.empty((T, n), dtype=torch.float32, device=proj.device)
-            library.call("ra_gla_chunks", *head, cum.data_ptr(), *tail)
+            scratch = self._chunk_scratch(T, batch.num_seqs, heads, key_dim, value_dim, proj.device)
+            library.call("ra_gla_chunks", *head, *tail, *sizes, scratch.data_ptr(), scratch.numel(), out.data_ptr(), _stream())
         else:
-            library.call("ra_gla_scan", *head, *tail)
+            library.call("ra_gla_scan", *head, *tail, longest, *sizes, out.data_ptr(), _stream())
 
     # -------------------------------------------------------------- several residual streams
     def hyper_step(self, streams: torch.Tensor, base: Optional[torch.Tensor], y: Optional[torch.Tensor],
