@@ -15,7 +15,7 @@
 // the factors; it leaves B_i q_i, (B_C / B_j) k_j, B_C, v and a as floats in the order in which the products want them.
 // chunk_carry_kernel walks a request's chunks with nothing left to do but those products: a workgroup is one (request,
 // head, 16 columns of v), its waves (four, or eight for keys above 64) split dk, the state stays in their accumulators
-// from the portion's first chunk to its last, operands come straight from memory, two chunks ahead.
+// from the portion's first chunk to its last, operands come straight from memory, CS_AHEAD chunks ahead.
 //
 // Everything is float: the products are v_mfma_f32_16x16x4_f32. The accumulator of a 16 x 16 product (row 4 g + i, column
 // r in lane 16 g + r, register i) is at the same time the operand of a product over those rows, if step i of four takes
@@ -32,6 +32,7 @@ namespace {
 
 #define CS_C 16                 // tokens of a chunk
 #define CS_VP 20                // floats between rows of the waves' parts in LDS
+#define CS_AHEAD 4              // chunks whose operands are on their way (a multiple of 4)
 #define CS_LIMIT 60.f           // -log2 of the smallest factor that the product form of the scores takes
 
 enum { CS_SILU = 0, CS_TURN = 1, CS_CHANNEL = 2 };       // silu on q, k, v; rotation and factors; a decay a key channel
@@ -290,11 +291,11 @@ __global__ void __launch_bounds__(WAVES * RA_WAVE) chunk_carry_kernel(ChunkArgs 
   const ChunkLayout L = chunk_layout(DKP, p.dv);
   const size_t stride = (size_t)p.H * L.floats;      // from one chunk to the next
   const float* W = p.ops + (size_t)chunk_base(p.cu_tokens, seq) * stride + (size_t)head * L.floats;
-  const float* Wq = W + (size_t)wave * NT * 256 + lane * 4;
-  const float* Wk = Wq + L.k;
-  const float* Wb = W + L.b + wave * NT * 16 + 4 * g;
-  const float* Wv = W + L.v + (size_t)cg * 256 + lane * 4;
-  const float* Wa = W + L.a + (wave & 3) * RA_WAVE + lane;
+  // Operands and results go through buffer descriptors, and no memory access stands under a condition: a store past the
+  // descriptor's end is dropped, and with the same number of accesses on every path the waits for operands count exactly
+  // those asked for (under a condition the compiler waited for all of them: one trip to memory every two chunks).
+  const int q_at = (wave * NT * 256 + lane * 4) * 4, k_at = q_at + L.k * 4, b_at = (L.b + wave * NT * 16 + 4 * g) * 4;
+  const int v_at = (L.v + cg * 256 + lane * 4) * 4, a_at = (L.a + (wave & 3) * RA_WAVE + lane) * 4;
 
   // ---- the state: tile nt of the wave is rows base + 16 nt + 4 g + i, column r of the group
   const int base = wave * 16 * NT, col = cg * 16 + r;
@@ -303,7 +304,7 @@ __global__ void __launch_bounds__(WAVES * RA_WAVE) chunk_carry_kernel(ChunkArgs 
   float* st = p.state + (size_t)slot * p.slot_stride + ((size_t)head * p.waves_per_head + c_at / p.CPW) * p.wave_floats +
               (size_t)(c_at % p.CPW) * p.R;
   const bool from_zero = p.fresh[seq] != 0;
-  f32x4_t S[NT];
+  f32x4_t S[NT], S_last[NT];
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt)
 #pragma unroll
@@ -314,17 +315,19 @@ __global__ void __launch_bounds__(WAVES * RA_WAVE) chunk_carry_kernel(ChunkArgs 
 
   struct Operands { f32x4_t q[NT], k[NT], b[NT], v; float a; };
   auto load = [&](int c, Operands& x) {              // a chunk past the last reads the last one again
-    const size_t at = (size_t)min(c, n_chunks - 1) * stride;
+    const __amdgpu_buffer_rsrc_t rsrc = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<float*>(W + (size_t)min(c, n_chunks - 1) * stride), 0, L.floats * 4, 0x00020000);
+    auto four = [&](int at) { return __builtin_bit_cast(f32x4_t, __builtin_amdgcn_raw_buffer_load_b128(rsrc, at, 0, 0)); };
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt) {
-      x.q[nt] = *(const f32x4_t*)(Wq + at + nt * 256);
-      x.k[nt] = *(const f32x4_t*)(Wk + at + nt * 256);
-      x.b[nt] = *(const f32x4_t*)(Wb + at + nt * 16);
+      x.q[nt] = four(q_at + nt * 1024);
+      x.k[nt] = four(k_at + nt * 1024);
+      x.b[nt] = four(b_at + nt * 64);
     }
-    x.v = *(const f32x4_t*)(Wv + at);
-    x.a = Wa[at];
+    x.v = four(v_at);
+    x.a = __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(rsrc, a_at, 0, 0));
   };
-  auto step = [&](const Operands& x, float* part) {
+  auto step = [&](int c, const Operands& x, float* part) {
     f32x4_t o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt)
@@ -340,42 +343,60 @@ __global__ void __launch_bounds__(WAVES * RA_WAVE) chunk_carry_kernel(ChunkArgs 
       for (int i = 0; i < 4; ++i) S[nt][i] *= x.b[nt][i];
 #pragma unroll
       for (int i = 0; i < 4; ++i) S[nt] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.k[nt][i], x.v[i], S[nt], 0, 0, 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) S_last[nt][i] = c < n_chunks ? S[nt][i] : S_last[nt][i];      // a chunk past the last leaves no trace
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) part[wave * PART + (4 * g + i) * CS_VP + r] = o[i];
   };
-  Operands x0, x1;
-  load(0, x0);
-  load(1, x1);
-  int buf = 0;
-  for (int c = 0; c < n_chunks; c += 2) {
-    step(x0, red[buf][0]);
-    load(c + 2, x0);
-    if (c + 1 < n_chunks) {
-      step(x1, red[buf][1]);
-      load(c + 3, x1);
-    }
+  // where this thread's elements of two chunks' o go, in a window of rows that begins at the first of the two
+  int o_at[512 / THREADS];
+#pragma unroll
+  for (int u = 0; u < 512 / THREADS; ++u) {
+    const int idx = tid + u * THREADS, t = idx / 16, e = idx % 16;
+    o_at[u] = e < cols ? (int)((t * ow + e) * 4) : -1;
+  }
+  // two chunks a barrier; every set of operands is asked for CS_AHEAD chunks before its use
+  auto round = [&](int c, Operands& xa, Operands& xb, int buf) {
+    step(c, xa, red[buf][0]);
+    load(c + CS_AHEAD, xa);
+    __builtin_amdgcn_sched_barrier(0);               // the loads stay where they are asked for
+    step(c + 1, xb, red[buf][1]);
+    load(c + 1 + CS_AHEAD, xb);
+    __builtin_amdgcn_sched_barrier(0);
     __syncthreads();
     // a thread an element of o: the waves' parts in order. The next round writes the other buffer, and the one after it
     // this one again, behind a barrier that every thread reaches only after its reads here.
-    for (int idx = tid; idx < 2 * 256; idx += THREADS) {
-      const int t = idx / 16, e = idx % 16, row = first + c * CS_C + t;
-      if (row < last && e < cols) {
-        const float* part = red[buf][t / CS_C] + (t % CS_C) * CS_VP + e;
-        float s = 0.f;
+    const int row0 = min(first + c * CS_C, last), rows = min(2 * CS_C, last - row0);
+    const __amdgpu_buffer_rsrc_t rsrc =
+        __builtin_amdgcn_make_buffer_rsrc(out + (size_t)row0 * ow, 0, (int)(rows * ow * 4), 0x00020000);
 #pragma unroll
-        for (int w = 0; w < WAVES; ++w) s += part[w * PART];
-        out[(size_t)row * ow + e] = s;
-      }
+    for (int u = 0; u < 512 / THREADS; ++u) {
+      const int idx = tid + u * THREADS, t = idx / 16, e = idx % 16;
+      const float* part = red[buf][t / CS_C] + (t % CS_C) * CS_VP + e;
+      float s = 0.f;
+#pragma unroll
+      for (int w = 0; w < WAVES; ++w) s += part[w * PART];
+      __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(unsigned, s), rsrc, o_at[u], 0, 0);
     }
-    buf ^= 1;
+  };
+  Operands x[CS_AHEAD];
+#pragma unroll
+  for (int k = 0; k < CS_AHEAD; ++k) {
+    load(k, x[k]);
+    __builtin_amdgcn_sched_barrier(0);
+  }
+  for (int c = 0; c < n_chunks; c += CS_AHEAD) {
+#pragma unroll
+    for (int k = 0; k < CS_AHEAD; k += 2)
+      round(c + k, x[k], x[k + 1], (k >> 1) & 1);
   }
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int e = base + 16 * nt + 4 * g + i;
-      if (col_ok && e < p.R * p.NPL) st[(size_t)(e % p.NPL) * RA_WAVE + e / p.NPL] = S[nt][i];
+      if (col_ok && e < p.R * p.NPL) st[(size_t)(e % p.NPL) * RA_WAVE + e / p.NPL] = S_last[nt][i];
     }
 }
 
@@ -388,6 +409,7 @@ int chunk_run(const ChunkArgs& a, const char* what, hipStream_t stream) {
   RA_CHECK(places <= 0x7fffffffL && units <= 0x7fffffffL, "%s: too many workgroups", what);
   const size_t lds = (size_t)(CS_C * (a.dkp + 4) * (MODE == CS_CHANNEL ? 3 : 2) + 4 * CS_C * CS_VP) * sizeof(float);
   RA_CHECK(lds <= 64 * 1024, "%s: %zu bytes of LDS", what, lds);
+  RA_CHECK((long)a.H * a.dv * 2 * CS_C * 4 < (1L << 31), "%s: rows of %ld floats", what, (long)a.H * a.dv);
   chunk_prepare_kernel<TA, MODE><<<(unsigned)places, 256, lds, stream>>>(a);
   RA_LAUNCH_CHECK(what);
   if (a.dkp == 64) chunk_carry_kernel<1, 4><<<(unsigned)units, 4 * RA_WAVE, 0, stream>>>(a);
