@@ -5,7 +5,7 @@ Keys and values live in blocks of ``block_size`` tokens. Layers with the same
 needs form a group (all earlier keys, or a window of them); every group has a
 pool of its own and every request has one block table per group. Blocks are
 taken lazily, when a step's tokens need them, given back when the request ends
-or, in a window group, when the window has passed them, and used again, last
+or, in a window group, when the window (or the chunk) has passed them, and used again, last
 freed first (the reference's ``PagePool`` is LIFO the same way,
 crates/memory/src/pool.rs:61-155). Beside the pools there are slots for
 per-request state of fixed size (one id per live request).
@@ -30,20 +30,23 @@ class CacheGroupSpec:
     window: int
     entries: Tuple[int, ...]
     keep: int = 0           # a window's first tokens that stay in sight: their blocks are never given back before the end
+    chunked: bool = False   # the window is the query's chunk of that many tokens: whole chunks are given back
 
 
-def plan_groups(windows: Sequence[Optional[int]], keeps: Optional[Sequence[int]] = None) -> List[CacheGroupSpec]:
+def plan_groups(windows: Sequence[Optional[int]], keeps: Optional[Sequence[int]] = None,
+                chunked: Optional[Sequence[bool]] = None) -> List[CacheGroupSpec]:
     """Group run-order entries by what they keep.
 
     ``windows[i]`` is None for an entry without keys of its own (it reads
     another entry's cache, or keeps fixed-size state), 0 for all keys, W > 0 for
     a window; ``keeps[i]`` is how many first tokens such a window keeps in sight
-    (none given: 0). Entries with equal needs share a group.
+    (none given: 0), ``chunked[i]`` whether it is a chunk counted from position 0 (none given: no).
+    Entries with equal needs share a group.
     """
-    by: Dict[Tuple[int, int], List[int]] = {}
+    by: Dict[Tuple[int, int, bool], List[int]] = {}
     for i, w in enumerate(windows):
         if w is None:
             continue
         keep = int(keeps[i]) if keeps is not None and w else 0
-        by.setdefault((int(w), keep), []).append(i)
-    return [CacheGroupSpec(window=w, entries=tuple(es), keep=k) for (w, k), es in sorted(by.items())]
+        by.setdefault((int(w), keep, bool(chunked[i]) if chunked is not None and w else False), []).append(i)
+    return [CacheGroupSpec(window=w, entries=tuple(es), keep=k, chunked=c) for (w, k, c), es in sorted(by.items())]

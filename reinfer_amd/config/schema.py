@@ -98,11 +98,24 @@ class NormSpec:
 
 
 @dataclass(frozen=True)
+class YarnSpec:
+    """A rotation's frequencies fitted to longer contexts (``PositionSpec.scaling``): with
+    dim(t) = n ln(original / (2 pi t)) / (2 ln theta) over the n entries turned, pairs below floor(dim(fast)) keep their
+    frequency, those above ceil(dim(slow)) have it divided by ``factor``, those between go over linearly; sine and cosine are
+    multiplied by 0.1 ln(factor) + 1."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
 class PositionSpec:
     kind: str            # e.g. "rope_neox"; "none" for no position encoding
     rotary_dim: int = 0
     theta: float = 10000.0
     extra: Tuple[Tuple[str, Any], ...] = ()   # for position parts defined elsewhere
+    scaling: Optional[YarnSpec] = None        # of the frequencies; None: as they are
 
     def option(self, name: str, default: Any = None) -> Any:
         return dict(self.extra).get(name, default)
@@ -137,6 +150,10 @@ class MixerSpec:
     keep_first: int = 0             # with a window: a request's first tokens that stay in sight
     values_are_keys: bool = False   # no value tensors: a value is the key as projected, before norm and rotation
     out_bias: bool = False          # the output projection has a bias
+    qk_norm_weights: bool = True    # False: the per-head norm of q and k has no weights
+    chunked: bool = False           # the window is the query's own chunk of that many keys, counted from position 0
+    sink: bool = False              # one more term exp(s_h) in the softmax's denominator, a number a query head
+    head_gate: bool = False         # a head's result times sigmoid(W_g h)_h, one number a head, before the output projection
 
     def option(self, name: str, default: Any = None) -> Any:
         return dict(self.extra).get(name, default)

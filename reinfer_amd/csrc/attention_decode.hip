@@ -87,7 +87,8 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
                     const int* __restrict__ token_list, const int* __restrict__ seq_of_token,
                     const int* __restrict__ positions, int block_size, int Hkv, int G, int d_arg,
                     float scale_log2, int window, int keep, int chunk_shift, int max_chunks, int n_tokens,
-                    int t_base, float* __restrict__ part_o, float* __restrict__ part_ml, float scale, RaScoreMod mod) {
+                    int t_base, float* __restrict__ part_o, float* __restrict__ part_ml, float scale, RaScoreMod mod,
+                    int aligned, RaHeadOut ho) {
   constexpr bool MOD = (FLAGS & FD_MOD) != 0, KEEP = (FLAGS & FD_KEEP) != 0;
   constexpr int FD_THREADS = FD_WAVES * RA_WAVE;
   const int d = EXACT ? DMAX : d_arg;
@@ -110,7 +111,7 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
     // seq_of_token null: every request of the step brings one token, token t is request t
     const int seq = seq_of_token ? seq_of_token[t] : t;
     const int p = positions[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = ra_first_key(p, window, aligned);
     const int keep16 = KEEP ? fd_kept(keep, lo) : 0;
     const FdCut cut = fd_cut(p, lo, keep16, chunk_shift, max_chunks, FD_WAVES * 32);
     const int n_chunks = cut.n;
@@ -286,7 +287,9 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
         ot += lds_o[((size_t)w * G + h) * d + e] * c;
       }
       if (n_chunks == 1) {
-        out[(size_t)t * out_stride + (size_t)(kvh * G + h) * d + e] = from_f32<bf16_t>(ot / lt);
+        const int head = kvh * G + h;
+        lt += ra_sink_term(ho, head, mw);
+        out[(size_t)t * out_stride + (size_t)head * d + e] = from_f32<bf16_t>(ot / lt * ra_head_gate<bf16_t>(ho, t, head));
       } else {
         part_o[(prow + h) * d + e] = ot;
         if (e == 0) {
@@ -311,7 +314,7 @@ __global__ void __launch_bounds__(RA_WAVE)
 flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                           bf16_t* __restrict__ out, int out_stride, const int* __restrict__ token_list,
                           const int* __restrict__ positions, int Hkv, int G, int d, int window, int keep, int chunk_shift,
-                          int max_chunks, int gran, int t_base) {
+                          int max_chunks, int gran, int t_base, int aligned, RaHeadOut ho) {
   const int head = blockIdx.x, li = blockIdx.y;
   const int lane = threadIdx.x;
   const int kvh = head / G, h = head % G;
@@ -334,14 +337,14 @@ flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restr
       }
     }
     const int p = positions[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = ra_first_key(p, window, aligned);
     const int n_chunks = fd_cut(p, lo, fd_kept(keep, lo), chunk_shift, max_chunks, gran).n;
     if (n_chunks == 1) return;                           // written by the first kernel
     const bool mine = lane < n_chunks;
     const float mc = mine ? mc_raw : -INFINITY, lc = mine ? lc_raw : 0.f;
     const float mt = wave_max(mc);                       // finite: every chunk saw at least one key
     const float w = mine ? fd_exp2(mc - mt) : 0.f;
-    const float lt = wave_sum(lc * w);
+    const float lt = wave_sum(lc * w) + ra_sink_term(ho, head, mt);
     float acc[EPL];
 #pragma unroll
     for (int i = 0; i < EPL; ++i) acc[i] = 0.f;
@@ -353,7 +356,7 @@ flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restr
         for (int i = 0; i < EPL; ++i) acc[i] += v[c][i] * wc;
       }
     }
-    const float inv = 1.f / lt;
+    const float inv = ra_head_gate<bf16_t>(ho, t, head) / lt;
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
       const int e = lane + i * RA_WAVE;
@@ -362,7 +365,7 @@ flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restr
     return;
   }
   const int p = positions[t];
-  const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+  const int lo = ra_first_key(p, window, aligned);
   const int n_chunks = fd_cut(p, lo, fd_kept(keep, lo), chunk_shift, max_chunks, gran).n;
   if (n_chunks == 1) return;                           // written by the first kernel
   float acc[4] = {0.f, 0.f, 0.f, 0.f};                 // d <= 256: up to 4 outputs a lane
@@ -402,7 +405,7 @@ flash_decode_merge_kernel(const float* __restrict__ part_o, const float* __restr
         for (int i = 0; i < 4; ++i) acc[i] += v[u][i] * wc[u];
     }
   }
-  const float inv = 1.f / lt;
+  const float inv = ra_head_gate<bf16_t>(ho, t, head) / (lt + ra_sink_term(ho, head, mt));
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int e = lane + i * RA_WAVE;
@@ -493,22 +496,27 @@ extern "C" int ra_attention_decode(const void* q, int q_stride, void* out, int o
                                    int d, float scale, int window, int chunk, int max_chunks, int waves,
                                    float* part_o, float* part_ml, hipStream_t stream) {
   return ra_attention_decode_mod(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, token_list,
-                                 seq_of_token, positions, n_tokens, block_size, Hq, Hkv, d, scale, window, 0, chunk,
-                                 max_chunks, waves, part_o, part_ml, 0.f, nullptr, nullptr, stream);
+                                 seq_of_token, positions, n_tokens, block_size, Hq, Hkv, d, scale, window, 0, 0, chunk,
+                                 max_chunks, waves, part_o, part_ml, 0.f, nullptr, nullptr, nullptr, nullptr, 0, stream);
 }
 
 // The same with the scores changed before the softmax: softcap > 0 caps them by a tanh, r1 / r2 (one float a query
-// head each; both or neither) take r1 ln(1 + r2 (position - key)) off.
+// head each; both or neither) take r1 ln(1 + r2 (position - key)) off. aligned: the window is the query's chunk; sink
+// and gate as in RaHeadOut.
 extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, int out_stride,
                                        const void* kcache, const void* vcache, const int* block_tables,
                                        int max_blocks, const int* token_list, const int* seq_of_token,
                                        const int* positions, int n_tokens, int block_size, int Hq, int Hkv,
-                                       int d, float scale, int window, int keep, int chunk, int max_chunks, int waves,
-                                       float* part_o, float* part_ml, float softcap, const float* r1,
-                                       const float* r2, hipStream_t stream) {
+                                       int d, float scale, int window, int aligned, int keep, int chunk, int max_chunks,
+                                       int waves, float* part_o, float* part_ml, float softcap, const float* r1,
+                                       const float* r2, const float* sink, const void* gate, int gate_stride,
+                                       hipStream_t stream) {
   RA_CHECK((r1 == nullptr) == (r2 == nullptr) && softcap >= 0.f,
            "attention_decode: the distance term takes both per-head vectors, the cap is not negative");
+  RA_CHECK(gate == nullptr || gate_stride >= Hq, "attention_decode: gate rows of %d for %d heads", gate_stride, Hq);
+  RA_CHECK(!aligned || keep == 0, "attention_decode: chunks keep no first keys");
   const RaScoreMod mod = {softcap, r1, r2};
+  const RaHeadOut ho = {sink, gate, gate_stride};
   const bool changed = softcap > 0.f || r1 != nullptr;
   RA_CHECK(n_tokens > 0, "attention_decode: no tokens");
   RA_CHECK(ra_attention_decode_supports(Hq, Hkv, d, block_size),
@@ -539,7 +547,7 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
 #define RA_FD_ARGS                                                                                    \
   (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache, (const bf16_t*)vcache, \
       block_tables, max_blocks, token_list, seq_of_token, positions, block_size, Hkv, G, d, scale_log2, \
-      window, keep, chunk_shift, max_chunks, n_tokens, 0, part_o, part_ml, scale, mod
+      window, keep, chunk_shift, max_chunks, n_tokens, 0, part_o, part_ml, scale, mod, aligned, ho
 #define RA_FD_GO(DM, EX, WV)                                                                          \
   do {                                                                                                \
     if (fd_allow_lds<DM, EX, WV>(lds) != hipSuccess)                                                  \
@@ -571,7 +579,8 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
     dim3 mg(Hq, n_tokens);
 #define RA_FDM(AH)                                                                                          \
   flash_decode_merge_kernel<AH><<<mg, RA_WAVE, 0, stream>>>(part_o, part_ml, (bf16_t*)out, out_stride, token_list, \
-                                                           positions, Hkv, G, d, window, keep, chunk_shift, max_chunks, waves * 32, 0)
+                                                           positions, Hkv, G, d, window, keep, chunk_shift, max_chunks, waves * 32, 0, \
+                                                           aligned, ho)
     if (max_chunks > FDM_AHEAD) RA_FDM(0);
     else if (d <= 64) RA_FDM(1);
     else if (d <= 128) RA_FDM(2);

@@ -4,12 +4,14 @@
 // weighted sum of values are float.
 //
 //   s_t = scale * (q . K_t) for keys t in [lo, p] of the token's own request,
-//   lo = max(0, p - window + 1) if window > 0 else 0; softmax with the running
+//   lo = max(0, p - window + 1) if window > 0 else 0 (aligned: the start of p's chunk of
+//   `window` keys); softmax with the running
 //   maximum subtracted; o = sum_t P_t V_t. With keep > 0 the first keep keys of the
 //   request are seen as well, however far the window has moved.
 //   Query head a reads KV head a / (Hq / Hkv).
 //   With a score change (RaScoreMod): s <- cap tanh(s / cap) where cap > 0, then
 //   s <- s - r1[a] ln(1 + r2[a] (p - t)) where the two per-head vectors are given.
+//   With a sink one more term exp(sink[a]) in the denominator, with a gate o times its sigmoid (RaHeadOut).
 // (crates/cuda/kernels/decode_gqa_kernels.cu:69-136; plain form
 //  crates/cuda/tests/engine_vs_cpu.rs:205-241)
 #include "common.h"
@@ -23,7 +25,8 @@ __global__ void attention_plain_kernel(const TA* __restrict__ q, int q_stride, T
                                        const int* __restrict__ token_list,
                                        const int* __restrict__ seq_of_token,
                                        const int* __restrict__ positions, int block_size, int Hq,
-                                       int Hkv, int d, float scale, int window, int keep, RaScoreMod mod) {
+                                       int Hkv, int d, float scale, int window, int aligned, int keep, RaScoreMod mod,
+                                       RaHeadOut ho) {
   extern __shared__ float lds[];          // q vector [d], then probabilities [64]
   float* qs = lds;
   float* ps = lds + d;
@@ -33,7 +36,7 @@ __global__ void attention_plain_kernel(const TA* __restrict__ q, int q_stride, T
   const int kvh = a / (Hq / Hkv);
   const int seq = seq_of_token[t];
   const int p = positions[t];
-  const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+  const int lo = ra_first_key(p, window, aligned);
   const int* table = block_tables + (size_t)seq * max_blocks;
   const TA* qv = q + (size_t)t * q_stride + (size_t)a * d;
   for (int i = lane; i < d; i += RA_WAVE) qs[i] = to_f32(qv[i]);
@@ -90,7 +93,8 @@ __global__ void attention_plain_kernel(const TA* __restrict__ q, int q_stride, T
     }
   }
   TA* o = out + (size_t)t * out_stride + (size_t)a * d;
-  const float inv = 1.f / l;
+  if (ho.sink) l += expf(ho.sink[a] - m);
+  const float inv = ra_head_gate<TA>(ho, t, a) / l;
 #pragma unroll
   for (int r = 0; r < 16; ++r) {
     if (r < n_acc) {
@@ -107,18 +111,21 @@ extern "C" int ra_attention_plain(const void* q, int q_stride, void* out, int ou
                                   int d, float scale, int window, hipStream_t stream) {
   return ra_attention_plain_mod(q, q_stride, out, out_stride, kcache, vcache, act_dtype, block_tables, max_blocks,
                                 token_list, seq_of_token, positions, n_tokens, block_size, Hq, Hkv, d, scale, window,
-                                0, 0.f, nullptr, nullptr, stream);
+                                0, 0, 0.f, nullptr, nullptr, nullptr, nullptr, 0, stream);
 }
 
 extern "C" int ra_attention_plain_mod(const void* q, int q_stride, void* out, int out_stride,
                                       const void* kcache, const void* vcache, int act_dtype,
                                       const int* block_tables, int max_blocks, const int* token_list,
                                       const int* seq_of_token, const int* positions, int n_tokens, int block_size,
-                                      int Hq, int Hkv, int d, float scale, int window, int keep, float softcap,
-                                      const float* r1, const float* r2, hipStream_t stream) {
+                                      int Hq, int Hkv, int d, float scale, int window, int aligned, int keep,
+                                      float softcap, const float* r1, const float* r2, const float* sink,
+                                      const void* gate, int gate_stride, hipStream_t stream) {
   RA_CHECK((r1 == nullptr) == (r2 == nullptr) && softcap >= 0.f,
            "attention_plain: the distance term takes both per-head vectors, the cap is not negative");
+  RA_CHECK(gate == nullptr || gate_stride >= Hq, "attention_plain: gate rows of %d for %d heads", gate_stride, Hq);
   const RaScoreMod mod = {softcap, r1, r2};
+  const RaHeadOut ho = {sink, gate, gate_stride};
   RA_CHECK(n_tokens > 0, "attention_plain: no tokens");
   RA_CHECK(Hq > 0 && Hkv > 0 && Hq % Hkv == 0, "attention_plain: %d query heads do not divide into %d groups", Hq, Hkv);
   RA_CHECK(d > 0 && d <= 1024, "attention_plain: head size %d outside 1..1024", d);
@@ -132,12 +139,12 @@ extern "C" int ra_attention_plain_mod(const void* q, int q_stride, void* out, in
   if (act_dtype == RA_F32)
     attention_plain_kernel<float><<<grid, RA_WAVE, lds, stream>>>(
         (const float*)q, q_stride, (float*)out, out_stride, (const float*)kcache, (const float*)vcache,
-        block_tables, max_blocks, token_list, seq_of_token, positions, block_size, Hq, Hkv, d, scale, window, keep, mod);
+        block_tables, max_blocks, token_list, seq_of_token, positions, block_size, Hq, Hkv, d, scale, window, aligned, keep, mod, ho);
   else if (act_dtype == RA_BF16)
     attention_plain_kernel<bf16_t><<<grid, RA_WAVE, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache,
         (const bf16_t*)vcache, block_tables, max_blocks, token_list, seq_of_token, positions, block_size,
-        Hq, Hkv, d, scale, window, keep, mod);
+        Hq, Hkv, d, scale, window, aligned, keep, mod, ho);
   else
     return ra_fail("attention_plain: unknown dtype tag %d", act_dtype);
   RA_LAUNCH_CHECK("attention_plain");

@@ -25,7 +25,8 @@
 // tile's exponentials.
 //
 // Causal: a query at position p sees keys <= p (and > p - window if a window is
-// set, but for the request's first `keep` keys, which a window may keep in sight). The reference's prompt attention is a vendored library kernel that sees
+// set, but for the request's first `keep` keys, which a window may keep in sight; or >= the start of p's own chunk of
+// `window` keys). The reference's prompt attention is a vendored library kernel that sees
 // only the prompt itself, from position 0 (crates/cuda/src/fmha.rs:574-686;
 // crates/cuda/kernels/fmha_kernels.cu:96); this one is written here and reads
 // earlier context from the cache, so a prompt can be cut anywhere.
@@ -72,7 +73,8 @@ struct FpSplit {
 // and changed score then replaces the product in the registers, and scale_log2 is log2(e) alone
 // FLAGS & FP_KEEP: a window that keeps the first `keep` keys; the rounds that hold them and lie below the window's
 // first round are walked before it.
-enum { FP_MOD = 1, FP_KEEP = 2 };
+// FLAGS & FP_CHUNK: the window is the query's own chunk of `window` keys, counted from position 0.
+enum { FP_MOD = 1, FP_KEEP = 2, FP_CHUNK = 4 };
 template <int DMAX, int NC, bool EXACT, int FLAGS>
 __global__ void __launch_bounds__(FP_THREADS)
 flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
@@ -80,8 +82,8 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
                      const int* __restrict__ block_tables, int max_blocks,
                      const int* __restrict__ tile_info,      // per tile: seq, first token row, n queries, first position
                      int block_size, int Hq, int Hkv, int d_arg, int HG, float scale_log2, int window,
-                     int keep, FpSplit sp, float mod_scale, RaScoreMod mod) {
-  constexpr bool MOD = (FLAGS & FP_MOD) != 0, KEEP = (FLAGS & FP_KEEP) != 0;
+                     int keep, FpSplit sp, float mod_scale, RaScoreMod mod, RaHeadOut ho) {
+  constexpr bool MOD = (FLAGS & FP_MOD) != 0, KEEP = (FLAGS & FP_KEEP) != 0, CHUNK = (FLAGS & FP_CHUNK) != 0;
   const int d = EXACT ? DMAX : d_arg;
   constexpr int NDT = DMAX / 32;       // 32-wide d tiles of the score product
   constexpr int NOT = DMAX / 16;       // 16-row d tiles of the output
@@ -123,11 +125,13 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
   const bool biased = MOD && mod.r1 != nullptr;
   const float inv_cap = (MOD && mod.softcap > 0.f) ? 1.f / mod.softcap : 0.f;
   float r1h[NC], r2h[NC];               // the distance term's two numbers of each column tile's head
+  int chunk_lo[NC];                     // CHUNK: the first key each column's query sees
 #pragma unroll
   for (int j = 0; j < NC; ++j) {
     const int c = wave * NC + j;
     qi[j] = (c / HG) * 16 + r;
     q_live[j] = qi[j] < nq && ((col_mask >> j) & 1);
+    chunk_lo[j] = CHUNK ? ra_first_key(pos0 + qi[j], window, 1) : 0;
     const int head = kvh * G + hgrp * HG + c % HG;
     r1h[j] = biased ? mod.r1[head] : 0.f;
     r2h[j] = biased ? mod.r2[head] : 0.f;
@@ -150,7 +154,7 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
 
   // keys this tile of queries can see, and this wave's share of them
   const int last_pos = pos0 + nq - 1;
-  const int first_key = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
+  const int first_key = ra_first_key(pos0, window, CHUNK ? 1 : 0);
   const int win_round = first_key / FP_KT * FP_KT;       // the round that holds the window's first key
   int kt_begin = win_round;
   int k_stop = last_pos;                      // the last key of this workgroup's rounds
@@ -178,6 +182,9 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
   const int w_qend = ((wave * NC + NC - 1) / HG + 1) * 16;      // one past its last
   const int w_first_pos = pos0 + w_q0;
   const int w_last_pos = pos0 + min(w_qend, nq) - 1;            // < w_first_pos if the wave has no query
+  // CHUNK: the first keys that the wave's first and last query see
+  const int w_first_lo = CHUNK ? ra_first_key(w_first_pos, window, 1) : 0;
+  const int w_last_lo = CHUNK ? ra_first_key(max(w_last_pos, w_first_pos), window, 1) : 0;
 
   // fetch of one round into registers: the four 16-slot tiles of K and of V, 16 bytes a thread and
   // step; tile tt_u of step u is the same for a whole wave, so its block id is a scalar load
@@ -258,7 +265,8 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
     const bf16_t* Vs = Vs2[buf];
     // a wave whose queries all lie before this round, or that has none, has nothing to add
     if (w_last_pos < w_first_pos || w_last_pos < k0) return;
-    if (window > 0 && k0 + FP_KT - 1 < w_first_pos - window + 1 && !(KEEP && k0 < keep)) return;
+    if (CHUNK ? k0 + FP_KT - 1 < w_first_lo
+              : window > 0 && k0 + FP_KT - 1 < w_first_pos - window + 1 && !(KEEP && k0 < keep)) return;
 
     // two halves of 32 keys, each: scores, online softmax, values
 #pragma unroll
@@ -334,12 +342,13 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
       }
       // keys strictly inside every query's view need no mask
       const bool inner = kh + 31 <= w_first_pos && w_qend <= nq &&
-                         (window <= 0 || kh >= w_last_pos - window + 1 || (KEEP && kh + 31 < keep));
+                         (CHUNK ? kh >= w_last_lo
+                                : window <= 0 || kh >= w_last_pos - window + 1 || (KEEP && kh + 31 < keep));
       if (!inner) {
 #pragma unroll
         for (int j = 0; j < NC; ++j) {
           const int q_pos = pos0 + qi[j];
-          const int q_lo = (window > 0 && q_pos - window + 1 > 0) ? q_pos - window + 1 : 0;
+          const int q_lo = CHUNK ? chunk_lo[j] : (window > 0 && q_pos - window + 1 > 0) ? q_pos - window + 1 : 0;
 #pragma unroll
           for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
@@ -467,8 +476,8 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
       continue;
     }
     if (!q_live[j]) continue;
-    const float inv = 1.f / lt;
     const int head = kvh * G + hgrp * HG + (wave * NC + j) % HG;
+    const float inv = ra_head_gate<bf16_t>(ho, row0 + qi[j], head) / (lt + ra_sink_term(ho, head, m[j]));
     bf16_t* op = out + (size_t)(row0 + qi[j]) * out_stride + (size_t)head * d;
 #pragma unroll
     for (int ot = 0; ot < NOT; ++ot) {
@@ -490,7 +499,7 @@ template <int DMAX>
 __global__ void __launch_bounds__(256)
 flash_prefill_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                            bf16_t* __restrict__ out, int out_stride, const int* __restrict__ merge_info,
-                           int gy, int n_hgrp, int G, int HG, int d, int n_cols) {
+                           int gy, int n_hgrp, int G, int HG, int d, int n_cols, RaHeadOut ho) {
   const int lane = threadIdx.x & (RA_WAVE - 1), wave = threadIdx.x / RA_WAVE;
   const int groups = n_cols / 4;                         // workgroups a (tile, KV head, head group): 4 columns each
   const int col = (blockIdx.x % groups) * 4 + wave;
@@ -520,7 +529,7 @@ flash_prefill_merge_kernel(const float* __restrict__ part_o, const float* __rest
         if (e < d) acc[i] += part_o[at * DMAX + e] * w;
       }
     }
-    const float inv = 1.f / lt;
+    const float inv = ra_head_gate<bf16_t>(ho, row0 + qi, head) / (lt + ra_sink_term(ho, head, mx));
     bf16_t* op = out + (size_t)(row0 + qi) * out_stride + (size_t)head * d;
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
@@ -556,7 +565,8 @@ flash_prefill_merge_kernel(const float* __restrict__ part_o, const float* __rest
 #pragma unroll
     for (int i = 0; i < EPL; ++i) acc[i] += v[p][i] * w;
   }
-  const float inv = 1.f / lt;                            // every query sees at least its own key
+  // every query sees at least its own key
+  const float inv = ra_head_gate<bf16_t>(ho, row0 + qi, head) / (lt + ra_sink_term(ho, head, mx));
   bf16_t* op = out + (size_t)(row0 + qi) * out_stride + (size_t)head * d;
 #pragma unroll
   for (int i = 0; i < EPL; ++i) {
@@ -599,17 +609,19 @@ extern "C" long ra_attention_prefill_part_floats(int Hq, int Hkv, int d, int n_s
 static int fp_launch(const void* q, int q_stride, void* out, int out_stride,
                      const void* kcache, const void* vcache, const int* block_tables,
                      int max_blocks, const int* tile_info, int n_tiles, int block_size,
-                     int Hq, int Hkv, int d, float scale, int window, int keep, const FpSplit& sp, const int* merge_info,
-                     int n_merge, const RaScoreMod& mod, hipStream_t stream) {
+                     int Hq, int Hkv, int d, float scale, int window, int aligned, int keep, const FpSplit& sp,
+                     const int* merge_info, int n_merge, const RaScoreMod& mod, const RaHeadOut& ho, hipStream_t stream) {
   RA_CHECK((mod.r1 == nullptr) == (mod.r2 == nullptr) && mod.softcap >= 0.f,
            "attention_prefill: the distance term takes both per-head vectors, the cap is not negative");
+  RA_CHECK(ho.gate == nullptr || ho.gate_stride >= Hq, "attention_prefill: gate rows of %d for %d heads", ho.gate_stride, Hq);
+  RA_CHECK(!aligned || keep == 0, "attention_prefill: chunks keep no first keys");
   const bool changed = mod.softcap > 0.f || mod.r1 != nullptr;
   RA_CHECK(n_tiles > 0, "attention_prefill: no query tiles");
   RA_CHECK(ra_attention_prefill_supports(Hq, Hkv, d, block_size),
            "attention_prefill: unsupported sizes (%d query heads, %d KV heads, head size %d, block %d)", Hq,
            Hkv, d, block_size);
   RA_CHECK(max_blocks > 0 && window >= 0 && keep >= 0, "attention_prefill: bad cache geometry");
-  if (window == 0) keep = 0;                      // without a window every key is seen
+  if (window == 0) keep = aligned = 0;            // without a window every key is seen
   RA_CHECK(q_stride % 8 == 0 && out_stride % 4 == 0 && ((uintptr_t)q % 16) == 0 && ((uintptr_t)out % 8) == 0 &&
                ((uintptr_t)kcache % 16) == 0 && ((uintptr_t)vcache % 16) == 0,
            "attention_prefill: operands must be 16-byte aligned");
@@ -622,10 +634,12 @@ static int fp_launch(const void* q, int q_stride, void* out, int out_stride,
   const float scale_log2 = (changed ? 1.f : scale) * 1.4426950408889634f;
 #define RA_FP_ARGS                                                                                    \
   (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache, (const bf16_t*)vcache, \
-      block_tables, max_blocks, tile_info, block_size, Hq, Hkv, d, sh.hg, scale_log2, window, keep, sp, scale, mod
+      block_tables, max_blocks, tile_info, block_size, Hq, Hkv, d, sh.hg, scale_log2, window, keep, sp, scale, mod, ho
 #define RA_FP_GO(DM, NCC, EX)                                                                         \
   do {                                                                                                \
-    if (changed && keep > 0) flash_prefill_kernel<DM, NCC, EX, FP_MOD | FP_KEEP><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
+    if (changed && aligned) flash_prefill_kernel<DM, NCC, EX, FP_MOD | FP_CHUNK><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
+    else if (aligned) flash_prefill_kernel<DM, NCC, EX, FP_CHUNK><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
+    else if (changed && keep > 0) flash_prefill_kernel<DM, NCC, EX, FP_MOD | FP_KEEP><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
     else if (changed) flash_prefill_kernel<DM, NCC, EX, FP_MOD><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
     else if (keep > 0) flash_prefill_kernel<DM, NCC, EX, FP_KEEP><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS); \
     else flash_prefill_kernel<DM, NCC, EX, 0><<<grid, FP_THREADS, 0, stream>>>(RA_FP_ARGS);           \
@@ -647,7 +661,7 @@ static int fp_launch(const void* q, int q_stride, void* out, int out_stride,
     RA_CHECK((long)n_merge * gy * (n_cols / 4) <= 0x7fffffffL, "attention_prefill: too many tiles to add up");
 #define RA_FPM(DM)                                                                                      \
   flash_prefill_merge_kernel<DM><<<n_merge * gy * (n_cols / 4), 256, 0, stream>>>(                      \
-      sp.part_o, sp.part_ml, (bf16_t*)out, out_stride, merge_info, gy, G / sh.hg, G, sh.hg, d, n_cols)
+      sp.part_o, sp.part_ml, (bf16_t*)out, out_stride, merge_info, gy, G / sh.hg, G, sh.hg, d, n_cols, ho)
     if (d <= 64) RA_FPM(64);
     else if (d <= 128) RA_FPM(128);
     else RA_FPM(256);
@@ -662,20 +676,24 @@ extern "C" int ra_attention_prefill(const void* q, int q_stride, void* out, int 
                                     int max_blocks, const int* tile_info, int n_tiles, int block_size,
                                     int Hq, int Hkv, int d, float scale, int window, hipStream_t stream) {
   return ra_attention_prefill_mod(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, tile_info,
-                                  n_tiles, block_size, Hq, Hkv, d, scale, window, 0, 0.f, nullptr, nullptr, stream);
+                                  n_tiles, block_size, Hq, Hkv, d, scale, window, 0, 0, 0.f, nullptr, nullptr, nullptr,
+                                  nullptr, 0, stream);
 }
 
 // The same with the scores changed before the softmax: softcap > 0 caps them by a tanh, r1 / r2 (one float a query
-// head each; both or neither) take r1 ln(1 + r2 (position - key)) off.
+// head each; both or neither) take r1 ln(1 + r2 (position - key)) off. aligned: the window is the query's chunk; sink
+// and gate as in RaHeadOut.
 extern "C" int ra_attention_prefill_mod(const void* q, int q_stride, void* out, int out_stride,
                                         const void* kcache, const void* vcache, const int* block_tables,
                                         int max_blocks, const int* tile_info, int n_tiles, int block_size,
-                                        int Hq, int Hkv, int d, float scale, int window, int keep, float softcap,
-                                        const float* r1, const float* r2, hipStream_t stream) {
+                                        int Hq, int Hkv, int d, float scale, int window, int aligned, int keep,
+                                        float softcap, const float* r1, const float* r2, const float* sink,
+                                        const void* gate, int gate_stride, hipStream_t stream) {
   const FpSplit none = {};
+  const RaHeadOut ho = {sink, gate, gate_stride};
   const RaScoreMod mod = {softcap, r1, r2};
   return fp_launch(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, tile_info, n_tiles,
-                   block_size, Hq, Hkv, d, scale, window, keep, none, nullptr, 0, mod, stream);
+                   block_size, Hq, Hkv, d, scale, window, aligned, keep, none, nullptr, 0, mod, ho, stream);
 }
 
 // The same with query tiles cut by keys: `ranges` holds three ints a listed tile (first key and one past the
@@ -690,15 +708,19 @@ extern "C" int ra_attention_prefill_split(const void* q, int q_stride, void* out
                                           hipStream_t stream) {
   return ra_attention_prefill_split_mod(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks,
                                         tile_info, n_tiles, ranges, merge_info, n_merge, part_o, part_ml, block_size,
-                                        Hq, Hkv, d, scale, window, 0, 0.f, nullptr, nullptr, stream);
+                                        Hq, Hkv, d, scale, window, 0, 0, 0.f, nullptr, nullptr, nullptr, nullptr, 0,
+                                        stream);
 }
 
 extern "C" int ra_attention_prefill_split_mod(const void* q, int q_stride, void* out, int out_stride,
                                               const void* kcache, const void* vcache, const int* block_tables,
                                               int max_blocks, const int* tile_info, int n_tiles, const int* ranges,
                                               const int* merge_info, int n_merge, float* part_o, float* part_ml,
-                                              int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
-                                              float softcap, const float* r1, const float* r2, hipStream_t stream) {
+                                              int block_size, int Hq, int Hkv, int d, float scale, int window,
+                                              int aligned, int keep, float softcap, const float* r1, const float* r2,
+                                              const float* sink, const void* gate, int gate_stride,
+                                              hipStream_t stream) {
+  const RaHeadOut ho = {sink, gate, gate_stride};
   const RaScoreMod mod = {softcap, r1, r2};
   RA_CHECK(ranges && merge_info && n_merge > 0 && part_o && part_ml,
            "attention_prefill_split: ranges, the list of cut tiles and the buffers for their parts are needed");
@@ -708,5 +730,5 @@ extern "C" int ra_attention_prefill_split_mod(const void* q, int q_stride, void*
   sp.part_o = part_o;
   sp.part_ml = part_ml;
   return fp_launch(q, q_stride, out, out_stride, kcache, vcache, block_tables, max_blocks, tile_info, n_tiles,
-                   block_size, Hq, Hkv, d, scale, window, keep, sp, merge_info, n_merge, mod, stream);
+                   block_size, Hq, Hkv, d, scale, window, aligned, keep, sp, merge_info, n_merge, mod, ho, stream);
 }

@@ -110,6 +110,32 @@ __device__ __forceinline__ float ra_mod_score_fast(float s, float softcap, float
   return s;
 }
 
+// ---- which keys a query sees, and what becomes of its sum over them ---------------------------------------------
+// The first key that a query at position p sees: 0 without a window; the last `window` keys; or, aligned, those of
+// its own chunk, the keys being cut into chunks of `window` from position 0 of the request.
+__device__ __forceinline__ int ra_first_key(int p, int window, int aligned) {
+  if (window <= 0) return 0;
+  if (aligned) return p - p % window;
+  return p - window + 1 > 0 ? p - window + 1 : 0;
+}
+// sink (float, one entry a query head): the softmax's denominator holds one more term, exp(sink[h]), which has no key
+// and no value; no scale, cap or distance term touches it. gate (of the activations' type, one number a token and query
+// head, rows gate_stride apart): the head's result is multiplied by its sigmoid.
+struct RaHeadOut {
+  const float* sink;
+  const void* gate;
+  int gate_stride;
+};
+// the sink's term beside sums taken against the maximum m of scores in powers of two
+__device__ __forceinline__ float ra_sink_term(const RaHeadOut& ho, int head, float m) {
+  return ho.sink ? __builtin_amdgcn_exp2f(ho.sink[head] * 1.4426950408889634f - m) : 0.f;
+}
+template <typename TA>
+__device__ __forceinline__ float ra_head_gate(const RaHeadOut& ho, int t, int head) {
+  if (!ho.gate) return 1.f;
+  return 1.f / (1.f + expf(-to_f32(((const TA*)ho.gate)[(size_t)t * ho.gate_stride + head])));
+}
+
 // ---- cache layout -----------------------------------------------------------
 // A block of the cache holds block_size (a multiple of 16) slots of one KV head
 // as block_size/16 tiles of 16 slots x d elements, 16*d elements each, laid out

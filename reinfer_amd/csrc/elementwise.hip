@@ -348,7 +348,7 @@ __global__ void qk_norm_rope_cache_kernel(TA* __restrict__ qkv, const TW* __rest
                                           const float* __restrict__ inv_freq, int rotary_dim,
                                           int rope_style, const int* __restrict__ slots,
                                           TA* __restrict__ kcache, TA* __restrict__ vcache,
-                                          int block_size, int Hq, int Hkv, int d, int v_back, QkSums sm) {
+                                          int block_size, int Hq, int Hkv, int d, int v_back, int ld, QkSums sm) {
   __shared__ float buf[QK_WAVES][QK_MAX_D];
   const int lane = threadIdx.x & (RA_WAVE - 1);
   const int wave = threadIdx.x / RA_WAVE;
@@ -360,7 +360,7 @@ __global__ void qk_norm_rope_cache_kernel(TA* __restrict__ qkv, const TW* __rest
   const bool is_k = !is_q && head < Hq + Hkv;
   const int row_heads = n_heads - v_back;
   const int src_head = (is_q || is_k) ? head : head - v_back;      // the head of the row that holds this one's elements
-  TA* u = qkv + ((size_t)t * row_heads + (live ? src_head : 0)) * d;
+  TA* u = qkv + (size_t)t * ld + (size_t)(live ? src_head : 0) * d;
   const int kvh = is_q ? 0 : (is_k ? head - Hq : head - Hq - Hkv);
   const int slot = slots[t];
   TA* slab = nullptr;           // the (block, kv head) slab a k or v head goes to
@@ -465,7 +465,7 @@ __global__ void __launch_bounds__(QK_WAVES * RA_WAVE)
 qk_norm_rope_cache_head_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w, const TW* __restrict__ k_w,
                                float eps, const int* __restrict__ positions, const float* __restrict__ inv_freq,
                                const int* __restrict__ slots, TA* __restrict__ kcache, TA* __restrict__ vcache,
-                               int block_size, int Hq, int Hkv, int v_back) {
+                               int block_size, int Hq, int Hkv, int v_back, int ld) {
   constexpr int d = 64 * EPL;
   constexpr int NF = EPL >= 2 ? EPL / 2 : 1;
   const int lane = threadIdx.x & (RA_WAVE - 1);
@@ -476,7 +476,7 @@ qk_norm_rope_cache_head_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w,
   if (head >= n_heads) return;
   const bool is_q = head < Hq;
   const bool is_k = !is_q && head < Hq + Hkv;
-  TA* u = qkv + ((size_t)t * (n_heads - v_back) + ((is_q || is_k) ? head : head - v_back)) * d;
+  TA* u = qkv + (size_t)t * ld + (size_t)((is_q || is_k) ? head : head - v_back) * d;
   const TW* w = is_q ? q_w : k_w;              // a v head reads k's weights and drops them
   // ---- every load, then the first use
   const int slot = slots[t];
@@ -598,7 +598,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
                                 float eps, const int* __restrict__ positions,
                                 const float* __restrict__ inv_freq, const int* __restrict__ slots,
                                 TA* __restrict__ kcache, TA* __restrict__ vcache, int block_size, int Hq,
-                                int Hkv, int d, int v_back, int T, int share) {
+                                int Hkv, int d, int v_back, int ld, int T, int share) {
   constexpr int E = Row16<TA>::E;
   constexpr int ROWS = 256 / LPH;              // head rows a pass of the workgroup
   extern __shared__ __attribute__((aligned(16))) unsigned char qk_lds[];
@@ -612,7 +612,6 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
   const int w_xcd = blockIdx.x % RA_XCDS, w_k = blockIdx.x / RA_XCDS;
   const int t = ((w_k / 16) * RA_XCDS + w_xcd) * 16 + w_k % 16;
   if (t >= T) return;
-  const int n_heads = Hq + 2 * Hkv - v_back;   // heads of a row
   const int sub = threadIdx.x / LPH, ln = threadIdx.x % LPH;
   const int j0 = ln * E;                       // pairs j0..j0+E-1
   const int slot = slots[t];
@@ -622,7 +621,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
   // the first pass's query rows are asked for before anything they do not hang on is waited for
   f32x4_raw first_a = {}, first_c = {};
   if (sub < Hq) {
-    const TA* u = qkv + ((size_t)t * n_heads + sub) * d;
+    const TA* u = qkv + (size_t)t * ld + (size_t)sub * d;
     first_a = *(const f32x4_raw*)(u + j0);
     first_c = *(const f32x4_raw*)(u + half + j0);
   }
@@ -674,7 +673,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
 
   // the token's own query heads, in place
   for (int head = sub; head < Hq; head += ROWS) {
-    TA* u = qkv + ((size_t)t * n_heads + head) * d;
+    TA* u = qkv + (size_t)t * ld + (size_t)head * d;
     float ra[E], rc[E];
     if (head == sub) turn_held(first_a, first_c, q_w, me, ra, rc);
     else turn(u, q_w, me, ra, rc);
@@ -689,7 +688,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
     for (int r = sub; r < 2 * Hkv; r += ROWS) {
       const bool is_k = r < Hkv;
       const int kvh = is_k ? r : r - Hkv;
-      const TA* u = qkv + ((size_t)t * n_heads + Hq + (is_k ? r : r - v_back)) * d;
+      const TA* u = qkv + (size_t)t * ld + (size_t)(Hq + (is_k ? r : r - v_back)) * d;
       TA* slab = (is_k ? kcache : vcache) + (blk * Hkv + kvh) * (size_t)block_size * d;
       if (is_k) {                              // the elements of one 8-chunk are contiguous in the K tile
         float ra[E], rc[E];
@@ -721,7 +720,7 @@ qk_norm_rope_cache_token_kernel(TA* __restrict__ qkv, const TW* __restrict__ q_w
     const int m = r >> 3, tok = r & 3;
     const bool is_k = (r & 4) == 0;
     const int kvh = me + 4 * m;
-    const TA* u = qkv + ((size_t)(t0 + tok) * n_heads + Hq + (is_k ? 0 : Hkv - v_back) + kvh) * d;
+    const TA* u = qkv + (size_t)(t0 + tok) * ld + (size_t)(Hq + (is_k ? 0 : Hkv - v_back) + kvh) * d;
     if (is_k) {
       float ra[E], rc[E];
       turn(u, k_w, tok, ra, rc);
@@ -772,10 +771,10 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
                                    int weight_dtype, float eps, const int* positions,
                                    const float* inv_freq, int rotary_dim, int rope_style,
                                    const int* slots, void* kcache, void* vcache, int block_size,
-                                   int n_tokens, int Hq, int Hkv, int d, int values_are_keys, const QkSums& sm, hipStream_t stream) {
+                                   int n_tokens, int Hq, int Hkv, int d, int values_are_keys, int ld, const QkSums& sm, hipStream_t stream) {
   const int v_back = values_are_keys ? Hkv : 0;
   RA_CHECK(n_tokens > 0, "qk_norm_rope_cache: no tokens");
-  RA_CHECK(Hq > 0 && Hkv > 0 && d > 0, "qk_norm_rope_cache: bad head sizes (%d, %d, %d)", Hq, Hkv, d);
+  RA_CHECK(Hq > 0 && Hkv >= 0 && d > 0, "qk_norm_rope_cache: bad head sizes (%d, %d, %d)", Hq, Hkv, d);
   RA_CHECK(d <= QK_MAX_D, "qk_norm_rope_cache: head size %d above the supported %d", d, QK_MAX_D);
   RA_CHECK(rotary_dim >= 0 && rotary_dim <= d && rotary_dim % 2 == 0,
            "qk_norm_rope_cache: rotary width %d must be even and <= head size %d", rotary_dim, d);
@@ -784,12 +783,14 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
   RA_CHECK(block_size > 0 && block_size % 16 == 0 && d % 16 == 0,
            "qk_norm_rope_cache: the cache is tiled 16 x 16: block size %d and head size %d must be multiples of 16",
            block_size, d);
+  RA_CHECK(sm.parts || ld >= (Hq + 2 * Hkv - v_back) * d, "qk_norm_rope_cache: rows of %d do not hold the heads", ld);
   RA_CHECK(n_tokens <= 65535, "qk_norm_rope_cache: %d tokens in one launch (max 65535)", n_tokens);
   // the per-token kernel takes half-split rotation over the whole head, d in {16, 32, 64, 128, 256};
   // with few tokens (decode) a wave per head spreads over more of the chip (measured at 32 heads of 128:
   // 3.2 against 4.4 us at 64 tokens, 3.9 against 4.7 at 128, 6.2 against 5.4 at 255)
   const bool pow2 = (d & (d - 1)) == 0 && d >= 16 && d <= 256;
   if (!sm.parts && pow2 && n_tokens >= 192 && rope_style == 0 && rotary_dim == d && ((uintptr_t)qkv % 16) == 0 &&
+      ((long)ld * (act_dtype == RA_F32 ? 4 : 2)) % 16 == 0 &&
       (q_weight == nullptr || (((uintptr_t)q_weight % 16) == 0 && ((uintptr_t)k_weight % 16) == 0))) {
     // four tokens share their keys and values where the staging areas leave room for eight workgroups a CU
     const bool share = qk_token_lds(Hkv, d, act_dtype == RA_F32 ? 4 : 2, true) <= 16384;
@@ -798,7 +799,7 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
       <<<(n_tokens + 16 * RA_XCDS - 1) / (16 * RA_XCDS) * (16 * RA_XCDS), 256,                            \
          qk_token_lds(Hkv, d, sizeof(TA), share), stream>>>(                                              \
       (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, slots, (TA*)kcache,  \
-      (TA*)vcache, block_size, Hq, Hkv, d, v_back, n_tokens, share ? 1 : 0)
+      (TA*)vcache, block_size, Hq, Hkv, d, v_back, ld, n_tokens, share ? 1 : 0)
   /* lanes a head: 16 bytes of either half a lane (SH: 0 for 4-byte elements, 1 for 2-byte ones) */
 #define RA_TOK(TA, TW, SH)                           \
   do {                                               \
@@ -824,11 +825,11 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
     if (q_weight)                                                                                         \
       qk_norm_rope_cache_head_kernel<TA, TW, EPL, true><<<grid, QK_WAVES * RA_WAVE, 0, stream>>>(         \
           (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, slots, (TA*)kcache, \
-          (TA*)vcache, block_size, Hq, Hkv, v_back);                                                              \
+          (TA*)vcache, block_size, Hq, Hkv, v_back, ld);                                                              \
     else                                                                                                  \
       qk_norm_rope_cache_head_kernel<TA, TW, EPL, false><<<grid, QK_WAVES * RA_WAVE, 0, stream>>>(        \
           (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, slots, (TA*)kcache, \
-          (TA*)vcache, block_size, Hq, Hkv, v_back);                                                              \
+          (TA*)vcache, block_size, Hq, Hkv, v_back, ld);                                                              \
   } while (0)
 #define RA_HEAD(TA, TW)                      \
   do {                                       \
@@ -848,7 +849,7 @@ static int qk_norm_rope_cache_impl(void* qkv, int act_dtype, const void* q_weigh
 #define RA_GO(TA, TW)                                                                              \
   qk_norm_rope_cache_kernel<TA, TW><<<grid, QK_WAVES * RA_WAVE, 0, stream>>>(                      \
       (TA*)qkv, (const TW*)q_weight, (const TW*)k_weight, eps, positions, inv_freq, rotary_dim,   \
-      rope_style, slots, (TA*)kcache, (TA*)vcache, block_size, Hq, Hkv, d, v_back, sm)
+      rope_style, slots, (TA*)kcache, (TA*)vcache, block_size, Hq, Hkv, d, v_back, ld, sm)
   if (act_dtype == RA_F32 && weight_dtype == RA_F32) RA_GO(float, float);
   else if (act_dtype == RA_BF16 && weight_dtype == RA_BF16) RA_GO(bf16_t, bf16_t);
   else if (act_dtype == RA_BF16 && weight_dtype == RA_F32) RA_GO(bf16_t, float);
@@ -862,12 +863,12 @@ extern "C" int ra_qk_norm_rope_cache(void* qkv, int act_dtype, const void* q_wei
                                      int weight_dtype, float eps, const int* positions,
                                      const float* inv_freq, int rotary_dim, int rope_style,
                                      const int* slots, void* kcache, void* vcache, int block_size,
-                                     int n_tokens, int Hq, int Hkv, int d, int values_are_keys, hipStream_t stream) {
+                                     int n_tokens, int Hq, int Hkv, int d, int values_are_keys, int ld, hipStream_t stream) {
   RA_CHECK(qkv != nullptr, "qk_norm_rope_cache: no q/k/v rows");
   const QkSums none = {};
   return qk_norm_rope_cache_impl(qkv, act_dtype, q_weight, k_weight, weight_dtype, eps, positions, inv_freq,
                                  rotary_dim, rope_style, slots, kcache, vcache, block_size, n_tokens, Hq, Hkv, d,
-                                 values_are_keys, none, stream);
+                                 values_are_keys, ld, none, stream);
 }
 
 // The same from the float partial results of a product cut into K ranges ([n_ranges][n_tokens][width],
@@ -897,7 +898,7 @@ extern "C" int ra_qk_norm_rope_cache_sums(const float* parts, int n_ranges, cons
   sm.q_stride = q_stride;
   return qk_norm_rope_cache_impl(nullptr, act_dtype, q_weight, k_weight, weight_dtype, eps, positions, inv_freq,
                                  rotary_dim, rope_style, slots, kcache, vcache, block_size, n_tokens, Hq, Hkv, d,
-                                 values_are_keys, sm, stream);
+                                 values_are_keys, 0, sm, stream);
 }
 
 // ---------------------------------------------------------------------------

@@ -163,6 +163,7 @@ struct CacheManager {
   py::list groups;                             // the CacheGroupSpec records, as given
   std::vector<int> windows;
   std::vector<int> keeps;                      // per group: first tokens that a window keeps in sight (0: none)
+  std::vector<char> chunked;                   // per group: the window is the query's own chunk, counted from position 0
   int block_size;
   std::vector<BlockPool> pools;
   SlotPool slots;
@@ -176,6 +177,7 @@ struct CacheManager {
     for (auto g : groups) {
       windows.push_back(g.attr("window").cast<int>());
       keeps.push_back(py::hasattr(g, "keep") ? g.attr("keep").cast<int>() : 0);
+      chunked.push_back(py::hasattr(g, "chunked") && g.attr("chunked").cast<bool>() ? 1 : 0);
     }
     for (int n : num_blocks) pools.emplace_back(n);
   }
@@ -216,7 +218,7 @@ struct CacheManager {
   int first_needed_block(int g, int first_query_pos) const {
     const int w = windows[g];
     if (w <= 0) return 0;
-    const int lo = first_query_pos - w + 1;
+    const int lo = chunked[g] ? first_query_pos - first_query_pos % w : first_query_pos - w + 1;
     return std::max(0, lo) / block_size;
   }
   // Blocks that hold the first tokens which group g's window keeps in sight: held as long as the request lives.

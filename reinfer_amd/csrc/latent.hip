@@ -11,13 +11,19 @@
 // ---------------------------------------------------------------------------
 // One workgroup a token. proj row = [... q heads (each D unrotated | R rotated) ... | c_raw (rank) | kr (R) ...]
 //   c  = c_raw * rsqrt(mean(c_raw^2) + eps) * w
-//   rotation of the first rot_dims of an R-wide part: pair (i, i + rot_dims/2) by angle pos * inv_freq[i]
+//   rotation of the first rot_dims of an R-wide part: pair (i, i + rot_dims/2), or (2i, 2i + 1) where style is 1, by angle
+//   pos * inv_freq[i], sine and cosine times amp
 //   cache row (K and V layout alike) = [c | rot(kr) | 0 ...]            at slots[t] (-1: store nothing)
 //   q_lat[t, h, rank : Dp] = [rot(q_h rotated part) | 0 ...]            (columns below rank: head products)
 // ---------------------------------------------------------------------------
 template <typename TA>
-__device__ __forceinline__ float latent_rot(const TA* vec, int i, int half, int rot_dims, const float* cs,
+__device__ __forceinline__ float latent_rot(const TA* vec, int i, int half, int rot_dims, int style, const float* cs,
                                             const float* sn) {
+  if (style == 1) {
+    if (i >= rot_dims) return to_f32(vec[i]);
+    const float mine = to_f32(vec[i]) * cs[i >> 1], other = to_f32(vec[i ^ 1]) * sn[i >> 1];
+    return (i & 1) ? mine + other : mine - other;
+  }
   if (i < half) return to_f32(vec[i]) * cs[i] - to_f32(vec[i + half]) * sn[i];
   if (i < rot_dims) {
     const int j = i - half;
@@ -29,8 +35,8 @@ __device__ __forceinline__ float latent_rot(const TA* vec, int i, int half, int 
 template <typename TA, typename TW>
 __global__ void latent_prep_kernel(const TA* __restrict__ proj, int ld, int q_off, int dkv_off,
                                    const TW* __restrict__ cw, float eps, const int* __restrict__ positions,
-                                   const float* __restrict__ inv_freq, int rot_dims, int R, int rank, int H, int D,
-                                   TA* __restrict__ q_lat, int Dp, const int* __restrict__ slots,
+                                   const float* __restrict__ inv_freq, int rot_dims, int style, float amp, int R, int rank,
+                                   int H, int D, TA* __restrict__ q_lat, int Dp, const int* __restrict__ slots,
                                    TA* __restrict__ kcache, TA* __restrict__ vcache, int block_size) {
   extern __shared__ float sm[];          // cos [half], sin [half]
   __shared__ float red[17];
@@ -42,7 +48,12 @@ __global__ void latent_prep_kernel(const TA* __restrict__ proj, int ld, int q_of
   const TA* craw = row + dkv_off;
   const TA* kr = craw + rank;
   const float pos = (float)positions[t];
-  for (int j = threadIdx.x; j < half; j += blockDim.x) sincosf(pos * inv_freq[j], &sn[j], &cs[j]);
+  for (int j = threadIdx.x; j < half; j += blockDim.x) {
+    float s, c;
+    sincosf(pos * inv_freq[j], &s, &c);
+    sn[j] = s * amp;
+    cs[j] = c * amp;
+  }
   float ss = 0.f;
   for (int i = threadIdx.x; i < rank; i += blockDim.x) {
     const float v = to_f32(craw[i]);
@@ -58,7 +69,7 @@ __global__ void latent_prep_kernel(const TA* __restrict__ proj, int ld, int q_of
     for (int e = threadIdx.x; e < Dp; e += blockDim.x) {
       float v = 0.f;
       if (e < rank) v = to_f32(craw[e]) * rstd * to_f32(cw[e]);
-      else if (e < rank + R) v = latent_rot(kr, e - rank, half, rot_dims, cs, sn);
+      else if (e < rank + R) v = latent_rot(kr, e - rank, half, rot_dims, style, cs, sn);
       const TA o = from_f32<TA>(v);
       kb[cache_k_index(off, e, Dp)] = o;
       vb[cache_v_index(off, e, Dp)] = o;
@@ -69,17 +80,19 @@ __global__ void latent_prep_kernel(const TA* __restrict__ proj, int ld, int q_of
   for (int idx = threadIdx.x; idx < H * tail; idx += blockDim.x) {
     const int h = idx / tail, i = idx % tail;
     float v = 0.f;
-    if (i < R) v = latent_rot(row + q_off + (size_t)h * (D + R) + D, i, half, rot_dims, cs, sn);
+    if (i < R) v = latent_rot(row + q_off + (size_t)h * (D + R) + D, i, half, rot_dims, style, cs, sn);
     qo[(size_t)h * Dp + rank + i] = from_f32<TA>(v);
   }
 }
 
 extern "C" int ra_latent_prep(const void* proj, int act_dtype, int ld, int q_off, int dkv_off, const void* c_weight,
                               int weight_dtype, float eps, const int* positions, const float* inv_freq,
-                              int rot_dims, int R, int rank, int H, int D, void* q_lat, int Dp, const int* slots,
-                              void* kcache, void* vcache, int block_size, int n_tokens, hipStream_t stream) {
+                              int rot_dims, int rope_style, float amp, int R, int rank, int H, int D, void* q_lat,
+                              int Dp, const int* slots, void* kcache, void* vcache, int block_size, int n_tokens,
+                              hipStream_t stream) {
   RA_CHECK(n_tokens > 0 && H > 0 && D >= 0 && R >= 0 && rank > 0, "latent_prep: %d tokens, %d heads of %d + %d, rank %d",
            n_tokens, H, D, R, rank);
+  RA_CHECK(rope_style == 0 || rope_style == 1, "latent_prep: unknown rotation style %d", rope_style);
   RA_CHECK(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= R, "latent_prep: %d rotated of %d", rot_dims, R);
   RA_CHECK(Dp % 16 == 0 && Dp >= rank + R && block_size > 0 && block_size % 16 == 0,
            "latent_prep: cache rows of %d for rank %d + %d, blocks of %d", Dp, rank, R, block_size);
@@ -88,7 +101,8 @@ extern "C" int ra_latent_prep(const void* proj, int act_dtype, int ld, int q_off
   const size_t lds = (size_t)(rot_dims > 0 ? rot_dims : 2) * sizeof(float);
 #define RA_LP(TA, TW)                                                                                          \
   latent_prep_kernel<TA, TW><<<n_tokens, 256, lds, stream>>>(                                                  \
-      (const TA*)proj, ld, q_off, dkv_off, (const TW*)c_weight, eps, positions, inv_freq, rot_dims, R, rank, H, D, \
+      (const TA*)proj, ld, q_off, dkv_off, (const TW*)c_weight, eps, positions, inv_freq, rot_dims, rope_style, amp, R, \
+      rank, H, D,                                                                                              \
       (TA*)q_lat, Dp, slots, (TA*)kcache, (TA*)vcache, block_size)
   if (act_dtype == RA_F32 && weight_dtype == RA_F32) RA_LP(float, float);
   else if (act_dtype == RA_BF16 && weight_dtype == RA_BF16) RA_LP(bf16_t, bf16_t);

@@ -5,7 +5,7 @@
 #pragma once
 #include <hip/hip_runtime.h>
 
-#define RA_ABI_VERSION 24
+#define RA_ABI_VERSION 25
 
 #ifdef __cplusplus
 extern "C" {
@@ -29,7 +29,7 @@ int ra_add_group_rmsnorm(float* resid, const void* delta, const void* weight, in
 int ra_qk_norm_rope_cache(void* qkv, int act_dtype, const void* q_weight, const void* k_weight,
                           int weight_dtype, float eps, const int* positions, const float* inv_freq,
                           int rotary_dim, int rope_style, const int* slots, void* kcache, void* vcache,
-                          int block_size, int n_tokens, int Hq, int Hkv, int d, int values_are_keys,
+                          int block_size, int n_tokens, int Hq, int Hkv, int d, int values_are_keys, int ld,
                           hipStream_t stream);
 // The same from the partial results of ra_gemm_wide_partial (added here, in range order), optionally scaled
 // by the RMSNorm that product carried (in_ss [in_parts][n_tokens], eps, width); the rotated q goes to q_out.
@@ -39,7 +39,8 @@ int ra_qk_norm_rope_cache_sums(const float* parts, int n_ranges, const float* in
                                const float* inv_freq, int rotary_dim, int rope_style, const int* slots,
                                void* kcache, void* vcache, int block_size, int n_tokens, int Hq, int Hkv, int d,
                                int values_are_keys, hipStream_t stream);
-// values_are_keys: rows hold q and k heads alone, (Hq + Hkv) * d, and the cached value is the key before its norm
+// values_are_keys: rows hold q and k heads alone, (Hq + Hkv) * d, and the cached value is the key before its norm.
+// ld: elements from one row of qkv to the next (the heads stand at its start). Hkv 0: rows of q alone, nothing is cached.
 
 // gate_up is [T, 2I]: group == 0: gate columns [0, I), up columns [I, 2I); group > 0: gate and
 // up interleaved in runs of `group` columns (gate run, then the up run of the same features)
@@ -57,12 +58,16 @@ int ra_attention_plain(const void* q, int q_stride, void* out, int out_stride, c
 // The `_mod` forms of the three attention kernels change a score between the scaled product and the softmax:
 // softcap > 0: s <- softcap tanh(s / softcap); r1, r2 (float, one entry a query head, both or neither):
 // s <- s - r1[h] ln(1 + r2[h] (query position - key position)); the cap first. keep > 0 with a window: the request's
-// first keep keys are seen as well, however far the window has moved on.
+// first keep keys are seen as well, however far the window has moved on. aligned: a query sees the keys of its own chunk,
+// the keys being cut into chunks of `window` from position 0. sink (float, one entry a query head, or null): one more term
+// exp(sink[h]) in the softmax's denominator. gate (activations' type, gate[t * gate_stride + h], or null): a head's result
+// times its sigmoid.
 int ra_attention_plain_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                            const void* vcache, int act_dtype, const int* block_tables, int max_blocks,
                            const int* token_list, const int* seq_of_token, const int* positions, int n_tokens,
-                           int block_size, int Hq, int Hkv, int d, float scale, int window, int keep, float softcap,
-                           const float* r1, const float* r2, hipStream_t stream);
+                           int block_size, int Hq, int Hkv, int d, float scale, int window, int aligned, int keep,
+                           float softcap, const float* r1, const float* r2, const float* sink, const void* gate,
+                           int gate_stride, hipStream_t stream);
 // act 2 of ra_act_mul with its bound: g <- min(g, lim), u <- clamp(u, -lim, lim), out = g sigmoid(1.702 g) (u + 1)
 int ra_act_mul_bounded(const void* gate_up, void* out, int act_dtype, int n_tokens, int intermediate, int group,
                        int act, float lim, hipStream_t stream);
@@ -136,9 +141,10 @@ int ra_attention_decode(const void* q, int q_stride, void* out, int out_stride, 
 int ra_attention_decode_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                             const void* vcache, const int* block_tables, int max_blocks,
                             const int* token_list, const int* seq_of_token, const int* positions,
-                            int n_tokens, int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
-                            int chunk, int max_chunks, int waves, float* part_o, float* part_ml, float softcap,
-                            const float* r1, const float* r2, hipStream_t stream);
+                            int n_tokens, int block_size, int Hq, int Hkv, int d, float scale, int window,
+                            int aligned, int keep, int chunk, int max_chunks, int waves, float* part_o, float* part_ml,
+                            float softcap, const float* r1, const float* r2, const float* sink, const void* gate,
+                            int gate_stride, hipStream_t stream);
 int ra_attention_prefill_supports(int Hq, int Hkv, int d, int block_size);
 int ra_attention_prefill_tile(int Hq, int Hkv, int d);
 int ra_attention_prefill_columns(int Hq, int Hkv, int d);
@@ -160,13 +166,15 @@ int ra_attention_prefill_split(const void* q, int q_stride, void* out, int out_s
 
 int ra_attention_prefill_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                              const void* vcache, const int* block_tables, int max_blocks, const int* tile_info,
-                             int n_tiles, int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
-                             float softcap, const float* r1, const float* r2, hipStream_t stream);
+                             int n_tiles, int block_size, int Hq, int Hkv, int d, float scale, int window,
+                             int aligned, int keep, float softcap, const float* r1, const float* r2, const float* sink,
+                             const void* gate, int gate_stride, hipStream_t stream);
 int ra_attention_prefill_split_mod(const void* q, int q_stride, void* out, int out_stride, const void* kcache,
                                    const void* vcache, const int* block_tables, int max_blocks, const int* tile_info,
                                    int n_tiles, const int* ranges, const int* merge_info, int n_merge, float* part_o,
-                                   float* part_ml, int block_size, int Hq, int Hkv, int d, float scale, int window, int keep,
-                                   float softcap, const float* r1, const float* r2, hipStream_t stream);
+                                   float* part_ml, int block_size, int Hq, int Hkv, int d, float scale, int window,
+                                   int aligned, int keep, float softcap, const float* r1, const float* r2,
+                                   const float* sink, const void* gate, int gate_stride, hipStream_t stream);
 
 int ra_sample_slices(int vocab);
 int ra_sample(const float* logits, int n_rows, int vocab, int row_stride, const float* temperature,
@@ -222,10 +230,11 @@ int ra_tanh_cap(float* logits, int n_rows, int vocab, int row_stride, float cap,
 // proj rows hold H query heads ([D unrotated | R rotated] each) from column q_off and [c_raw (rank) | kr (R)] from
 // column dkv_off. Writes the cache row [rms(c_raw) * c_weight | rot(kr) | 0...] of Dp (a multiple of 16) elements in
 // the K and V tile layouts of one KV head at slots[t] (-1: nothing), and q_lat[t, h, rank:Dp] = [rot(q_h's rotated
-// part) | 0...]. Rotation: the first rot_dims of an R-wide part, half-split pairs, angle pos * inv_freq[i].
+// part) | 0...]. Rotation: the first rot_dims of an R-wide part, pairs half-split (rope_style 0) or of neighbours (1), angle
+// pos * inv_freq[i], sine and cosine times amp.
 int ra_latent_prep(const void* proj, int act_dtype, int ld, int q_off, int dkv_off, const void* c_weight,
-                   int weight_dtype, float eps, const int* positions, const float* inv_freq, int rot_dims, int R,
-                   int rank, int H, int D, void* q_lat, int Dp, const int* slots, void* kcache, void* vcache,
+                   int weight_dtype, float eps, const int* positions, const float* inv_freq, int rot_dims, int rope_style,
+                   float amp, int R, int rank, int H, int D, void* q_lat, int Dp, const int* slots, void* kcache, void* vcache,
                    int block_size, int n_tokens, hipStream_t stream);
 // out[t, h * o_head + n] = sum_k x[t, h * x_head + k] * W[h, k, n] (* sigmoid(gate[t, h * N + n]) if gate, or
 // * sigmoid(gate[t, h]) with gate_per_head: one number a head)

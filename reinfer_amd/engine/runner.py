@@ -16,7 +16,7 @@ from ..cache import CacheManager, OutOfBlocks, plan_groups
 from ..config import load_config
 from ..config.schema import ModelSpec
 from ..models import DecoderModel, declare_params
-from ..parts import JointNeed, KVNeed, LayerCache, PagedNeed, StateNeed, paged_need
+from ..parts import JointNeed, KVNeed, LayerCache, PagedNeed, StateNeed, covering, paged_need
 from ..weights import check_tensors, load_weights, random_tensor, random_tensors, storage_dtype, weight_from_folder
 from .._hostlib import StepError
 from .batch import StepBatch, StepEntry, build_step_batch
@@ -56,19 +56,27 @@ class ModelRunner:
         self.model = DecoderModel(spec, weights, dtype, device)
         needs = self.model.cache_needs()
 
+        # a layer that reads another's keys may see further back than that one: the pages are kept for both
+        for i, e in enumerate(spec.run_order):
+            src = e.cache_from
+            if src is not None and isinstance(needs[i], (KVNeed, PagedNeed)) and isinstance(needs[src], (KVNeed, PagedNeed)):
+                needs[src] = covering(needs[src], needs[i])
         # which run-order entries keep keys of their own, and with which window
         windows: List[Optional[int]] = []
         keeps: List[int] = []
+        chunked: List[bool] = []
         for e, need in zip(spec.run_order, needs):
             if paged_need(need) is not None and e.cache_from is None:
                 windows.append(paged_need(need).window)
                 keeps.append(int(getattr(paged_need(need), "keep", 0)))
+                chunked.append(bool(getattr(paged_need(need), "chunked", False)))
             else:
                 windows.append(None)
                 keeps.append(0)
+                chunked.append(False)
         # no layer with keys of its own: no group, no pool, no block tables; requests then hold a state
         # slot each and are admitted by slots alone
-        groups = plan_groups(windows, keeps)
+        groups = plan_groups(windows, keeps, chunked)
         self.groups = groups
         group_of = {i: g for g, gs in enumerate(groups) for i in gs.entries}
 

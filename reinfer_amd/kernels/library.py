@@ -15,7 +15,7 @@ import torch  # noqa: F401  (loads the HIP runtime the library links against)
 
 from ..csrc import build as _build
 
-ABI_VERSION = 24
+ABI_VERSION = 25
 
 
 class KernelLibraryError(RuntimeError):
@@ -31,7 +31,7 @@ P, I, F = c_void_p, c_int, c_float
 _SIGNATURES = {
     "ra_embed": [P, I, P, P, I, I, F, P],
     "ra_add_rmsnorm": [P, P, P, I, P, I, P, I, I, F, F, P],
-    "ra_qk_norm_rope_cache": [P, I, P, P, I, F, P, P, I, I, P, P, P, I, I, I, I, I, I, P],
+    "ra_qk_norm_rope_cache": [P, I, P, P, I, F, P, P, I, I, P, P, P, I, I, I, I, I, I, I, P],
     "ra_qk_norm_rope_cache_sums": [P, I, P, I, F, I, P, I, I, P, P, I, F, P, P, I, I, P, P, P, I, I, I, I, I, I, P],
     "ra_gemm_wide_partial": [P, P, P, c_long, I, I, I, I, P],
     "ra_silu_mul": [P, P, I, I, I, I, P],
@@ -52,7 +52,7 @@ _SIGNATURES = {
     "ra_pair_hash_add": [P, P, I, P, P, P, P, P, P, I, c_longlong, c_longlong, I, I, P],
     "ra_stream_add": [P, P, I, P, P, I, I, I, F, P],
     "ra_tanh_cap": [P, I, I, I, F, P],
-    "ra_latent_prep": [P, I, I, I, I, P, I, F, P, P, I, I, I, I, I, P, I, P, P, P, I, I, P],
+    "ra_latent_prep": [P, I, I, I, I, P, I, F, P, P, I, I, F, I, I, I, I, P, I, P, P, P, I, I, P],
     "ra_head_linear": [P, I, I, P, P, I, I, P, I, I, I, I, I, I, I, P],
     "ra_add_group_rmsnorm": [P, P, P, I, P, I, P, I, I, I, F, F, P],
     "ra_act_mul": [P, P, I, I, I, I, I, P],
@@ -77,10 +77,10 @@ _SIGNATURES = {
     "ra_delta_rule_scan": [P, I, P, P, P, P, c_long, P, P, P, I, I, I, I, I, I, I, P, P],
     "ra_head_norm_gate": [P, P, I, P, I, I, I, F, I, I, I, P, P],
     "ra_normed_mean": [P, P, I, I, F, I, I, P, P, F, P],
-    "ra_attention_plain_mod": [P, I, P, I, P, P, I, P, I, P, P, P, I, I, I, I, I, F, I, I, F, P, P, P],
-    "ra_attention_decode_mod": [P, I, P, I, P, P, P, I, P, P, P, I, I, I, I, I, F, I, I, I, I, I, P, P, F, P, P, P],
-    "ra_attention_prefill_mod": [P, I, P, I, P, P, P, I, P, I, I, I, I, I, F, I, I, F, P, P, P],
-    "ra_attention_prefill_split_mod": [P, I, P, I, P, P, P, I, P, I, P, P, I, P, P, I, I, I, I, F, I, I, F, P, P, P],
+    "ra_attention_plain_mod": [P, I, P, I, P, P, I, P, I, P, P, P, I, I, I, I, I, F, I, I, I, F, P, P, P, P, I, P],
+    "ra_attention_decode_mod": [P, I, P, I, P, P, P, I, P, P, P, I, I, I, I, I, F, I, I, I, I, I, I, P, P, F, P, P, P, P, I, P],
+    "ra_attention_prefill_mod": [P, I, P, I, P, P, P, I, P, I, I, I, I, I, F, I, I, I, F, P, P, P, P, I, P],
+    "ra_attention_prefill_split_mod": [P, I, P, I, P, P, P, I, P, I, P, P, I, P, P, I, I, I, I, F, I, I, I, F, P, P, P, P, I, P],
     "ra_act_mul_bounded": [P, P, I, I, I, I, I, F, P],
     "ra_decay_scan": [P, I, I, I, I, I, P, P, c_long, P, P, P, I, I, I, I, I, I, P, P],
     "ra_retention_scan": [P, I, I, I, I, I, P, P, P, I, F, F, P, c_long, P, P, P, I, I, I, I, I, I, P, P],

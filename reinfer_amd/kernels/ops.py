@@ -107,15 +107,18 @@ class HipKernels:
                            slots: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
                            num_heads: int, num_kv_heads: int, head_dim: int, values_are_keys: bool = False) -> None:
         """Head norm and rotation of q (in place) and k, k and v into the cache. ``values_are_keys``: the rows hold
-        q and k alone, and the value that is cached is the key as it stands there, before norm and rotation."""
+        q and k alone, and the value that is cached is the key as it stands there, before norm and rotation.
+        ``qkv`` may be wider than its heads (they stand at the start of a row). ``num_kv_heads`` 0: queries alone,
+        nothing is cached (``kcache`` and ``vcache`` None, ``k_weight`` as ``q_weight``)."""
         _dev(qkv, q_weight, k_weight, positions, inv_freq, slots, kcache, vcache)
         T = qkv.shape[0]
         width = (num_heads + (1 if values_are_keys else 2) * num_kv_heads) * head_dim
-        if qkv.shape != (T, width) or not qkv.is_contiguous():
-            raise ValueError(f"qk_norm_rope_cache: qkv {tuple(qkv.shape)}, expected [T, {width}] contiguous")
-        self._check_cache("qk_norm_rope_cache", kcache, vcache, num_kv_heads, head_dim)
-        if kcache.dtype != qkv.dtype or vcache.dtype != qkv.dtype:
-            raise TypeError("qk_norm_rope_cache: the cache has the activations' dtype")
+        if qkv.dim() != 2 or qkv.shape[1] < width or qkv.stride(1) != 1 or qkv.stride(0) < width:
+            raise ValueError(f"qk_norm_rope_cache: qkv {tuple(qkv.shape)}, expected rows of at least {width}")
+        if num_kv_heads:
+            self._check_cache("qk_norm_rope_cache", kcache, vcache, num_kv_heads, head_dim)
+            if kcache.dtype != qkv.dtype or vcache.dtype != qkv.dtype:
+                raise TypeError("qk_norm_rope_cache: the cache has the activations' dtype")
         _int32(positions, "positions", T)
         _int32(slots, "cache slots", T)
         if inv_freq.dtype != torch.float32 or inv_freq.numel() < rotary_dim // 2:
@@ -130,9 +133,9 @@ class HipKernels:
             raise TypeError("qk_norm_rope_cache: q and k norm weights differ in dtype")
         library.call("ra_qk_norm_rope_cache", qkv.data_ptr(), _tag(qkv, "qkv"), _ptr(q_weight),
                      _ptr(k_weight), wtag, float(eps), positions.data_ptr(), inv_freq.data_ptr(),
-                     int(rotary_dim), int(rope_style), slots.data_ptr(), kcache.data_ptr(),
-                     vcache.data_ptr(), kcache.shape[2] * 16, T, num_heads, num_kv_heads, head_dim,
-                     1 if values_are_keys else 0, _stream())
+                     int(rotary_dim), int(rope_style), slots.data_ptr(), _ptr(kcache) if num_kv_heads else None,
+                     _ptr(vcache) if num_kv_heads else None, kcache.shape[2] * 16 if num_kv_heads else 16, T, num_heads,
+                     num_kv_heads, head_dim, 1 if values_are_keys else 0, qkv.stride(0), _stream())
 
     # ---- the q/k/v product left in K ranges for the kernel that consumes it
     def linear_ranges(self, x: torch.Tensor, weight: torch.Tensor):
@@ -225,13 +228,16 @@ class HipKernels:
     def attention(self, q: torch.Tensor, q_stride: int, out: torch.Tensor, kcache: torch.Tensor,
                   vcache: torch.Tensor, batch, num_heads: int, num_kv_heads: int, head_dim: int,
                   scale: float, window: int, group: int, softcap: float = 0.0, distance=None,
-                  keep: int = 0) -> None:
+                  keep: int = 0, aligned: bool = False, sink=None, gate=None) -> None:
         """Attention of every token of the step over its request's cache.
 
         ``softcap`` > 0: score <- softcap * tanh(score / softcap); ``distance`` = (r1, r2), two float32 vectors
         with one entry a query head: score <- score - r1[h] * ln(1 + r2[h] * (query position - key position)),
         behind the cap. ``keep`` > 0 with a window: a request's first ``keep`` keys are seen as well, however far
-        the window has moved on. Every kernel below applies them alike.
+        the window has moved on. ``aligned``: the keys are cut into chunks of ``window`` from position 0 and a query
+        sees those of its own chunk alone. ``sink`` (float32, one entry a query head): the softmax's denominator holds
+        one more term exp(sink[h]). ``gate`` ([T, at least the query heads] rows of the activations' dtype, unit column
+        stride): a head's result is multiplied by the sigmoid of its number. Every kernel below applies them alike.
 
         ``q`` is the buffer whose row ``t`` holds the query heads of token t at
         its start (row stride ``q_stride`` elements); ``batch`` is the step's
@@ -249,6 +255,12 @@ class HipKernels:
             raise ValueError("attention: a negative number of kept keys")
         if keep and window:
             changed["keep"] = int(keep)
+        if aligned and window:
+            if keep:
+                raise ValueError("attention: chunks keep no first keys")
+            changed["aligned"] = True
+        if sink is not None or gate is not None:
+            changed["head_out"] = self._head_out(sink, gate, q, num_heads)
         if q.dtype != torch.bfloat16:
             return self.attention_plain(q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads,
                                         head_dim, scale, window, group, **changed)
@@ -261,7 +273,8 @@ class HipKernels:
         # query tile times the head size the kernel is built for
         cols = 128 * max(1, lib.ra_attention_prefill_columns(num_heads, num_kv_heads, head_dim))
         built_for = 64 if head_dim <= 64 else 128 if head_dim <= 128 else 256
-        plan = self._attention_plan(batch, q.device, tile, room, halves, (256 * 128) / (cols * built_for))
+        plan = self._attention_plan(batch, q.device, tile, room, halves, (256 * 128) / (cols * built_for),
+                                    int(window) if aligned else 0)
         dec_ok = bool(lib.ra_attention_decode_supports(num_heads, num_kv_heads, head_dim, bs))
         pre_ok = bool(lib.ra_attention_prefill_supports(num_heads, num_kv_heads, head_dim, bs))
         side = None
@@ -309,6 +322,17 @@ class HipKernels:
             if r.dtype != torch.float32 or r.shape != (num_heads,) or not r.is_contiguous() or r.device != device:
                 raise ValueError(f"attention: the distance term takes two float32 vectors of {num_heads} entries")
         return (float(softcap), r1.data_ptr(), r2.data_ptr())
+
+    @staticmethod
+    def _head_out(sink, gate, q, num_heads: int):
+        """(sink pointer or None, gate pointer or None, gate row stride) for the kernels' ``_mod`` entry points, checked."""
+        if sink is not None and (sink.dtype != torch.float32 or sink.shape != (num_heads,) or not sink.is_contiguous()
+                                 or sink.device != q.device):
+            raise ValueError(f"attention: the sink is a float32 vector of {num_heads} entries")
+        if gate is not None and (gate.dtype != q.dtype or gate.dim() != 2 or gate.shape[0] != q.shape[0]
+                                 or gate.shape[1] < num_heads or gate.stride(1) != 1 or gate.device != q.device):
+            raise ValueError(f"attention: the gate is [T, at least {num_heads}] in the queries' dtype, unit column stride")
+        return (_ptr(sink), _ptr(gate), gate.stride(0) if gate is not None else 0)
 
     def shared_head_limit(self, head_dim: int, block_size: int = 16) -> int:
         """Query heads that may share one KV head in a call of :meth:`attention` and still take the
@@ -361,7 +385,7 @@ class HipKernels:
             heapq.heappush(ends, heapq.heappop(ends) + c)
         return max(ends)
 
-    def _prefill_items(self, tiles, room: int, halves: bool, fixed: float = 1.0):
+    def _prefill_items(self, tiles, room: int, halves: bool, fixed: float = 1.0, chunk: int = 0):
         """The prompt kernel's work items for ``tiles`` of (request, row, queries, position), and the list
         for the kernel that adds the parts of tiles cut by keys: ``(items, merge, n_slots)``, an item being
         (cost, tile, first key, one past the last key, slot or -1).
@@ -377,11 +401,13 @@ class HipKernels:
         while there are fewer tiles than ``room``, the heaviest cut by keys into parts, each an item whose
         float sums a second kernel adds up; the spare room goes, one part at a time, to the tile whose
         parts are longest. (Windows are not known here, one plan serving all layers: a part below a
-        layer's window finds nothing to do.)"""
+        layer's window finds nothing to do. ``chunk`` > 0: the plan of layers whose queries see the keys of their own chunk
+        of that many alone; a tile's rounds then begin at the chunk of its first query.)"""
         R = self.PREFILL_ROUND
         n = len(tiles)
         item_cost = self.PREFILL_ITEM * fixed
-        rounds = [-(-(pos + q) // R) for (_, _, q, pos) in tiles]
+        begin = [pos // chunk * chunk // R if chunk else 0 for (_, _, _, pos) in tiles]      # a tile's first round
+        rounds = [-(-(pos + q) // R) - b for (_, _, q, pos), b in zip(tiles, begin)]
         whole = [(r + item_cost, tl, 0, 0, -1) for tl, r in zip(tiles, rounds)]
         if room <= 0 or n == 0:
             return whole, [], 0
@@ -430,8 +456,9 @@ class HipKernels:
                     continue
                 merge.extend((tl[1], tl[2], n_slots, p))
                 for j in range(p):
-                    hi = (j + 1) * per * R if j + 1 < p else 1 << 30
-                    items.append((min(per, r - j * per) + item_cost, tl, j * per * R, hi, n_slots + j))
+                    lo = (begin[k] + j * per) * R if j else 0
+                    hi = (begin[k] + (j + 1) * per) * R if j + 1 < p else 1 << 30
+                    items.append((min(per, r - j * per) + item_cost, tl, lo, hi, n_slots + j))
                 n_slots += p
             if n_slots:
                 span = self._span([it[0] for it in items], room) + (self.PREFILL_MERGE[0]
@@ -447,14 +474,15 @@ class HipKernels:
             "n_decode": num_rows, "decode_max_ctx": ctx_cap, "decode_list": None, "n_prefill": 0,
             "prefill_list": None, "n_tiles": 0, "tiles": None}
 
-    def _attention_plan(self, batch, device, tile: int, room: int = 0, halves: bool = False, fixed: float = 1.0):
+    def _attention_plan(self, batch, device, tile: int, room: int = 0, halves: bool = False, fixed: float = 1.0,
+                        chunk: int = 0):
         """Which tokens go to which kernel; made once per step and query-tile size, shared by the
         layers. ``room`` is the number of query tiles whose workgroups fill the chip once (0: the tiles
         are listed as they are)."""
         plan = batch.extra.get("attention_plan")
         if plan is not None and plan.get("tile", tile) == tile:
             return plan
-        plan = batch.extra.get(("attention_plan", tile, room, halves, fixed))
+        plan = batch.extra.get(("attention_plan", tile, room, halves, fixed, chunk))
         if plan is not None:
             return plan
         dec, pre, tiles = [], [], []
@@ -469,7 +497,7 @@ class HipKernels:
                 for q0 in range(0, ql, tile):
                     tiles.append((i, t + q0, min(tile, ql - q0), st + q0))
             t += ql
-        items, merge, n_slots = self._prefill_items(tiles, room, halves, fixed)
+        items, merge, n_slots = self._prefill_items(tiles, room, halves, fixed, chunk)
         items.sort(key=lambda it: it[0])                     # the heaviest last: the kernel starts the last listed first
         listed = [v for it in items for v in it[1]]
         ranges = [v for it in items for v in ((it[2], it[3], it[4]) if it[4] >= 0 else (0, 1 << 30, -1))] if merge else []
@@ -492,7 +520,7 @@ class HipKernels:
             "n_merge": len(merge) // 4, "n_slots": n_slots,
             "tile": tile,
         }
-        batch.extra[("attention_plan", tile, room, halves, fixed)] = plan
+        batch.extra[("attention_plan", tile, room, halves, fixed, chunk)] = plan
         return plan
 
     @staticmethod
@@ -526,7 +554,8 @@ class HipKernels:
         return tables
 
     def attention_plain(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
-                        scale, window, group, token_list=None, n_listed=None, mod=(0.0, None, None), keep: int = 0) -> None:
+                        scale, window, group, token_list=None, n_listed=None, mod=(0.0, None, None), keep: int = 0,
+                        aligned: bool = False, head_out=(None, None, 0)) -> None:
         tables = self._check_attention(q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads,
                                        head_dim, group)
         n = batch.num_tokens if token_list is None else int(n_listed)
@@ -534,7 +563,7 @@ class HipKernels:
                      kcache.data_ptr(), vcache.data_ptr(), _tag(q, "attention"), tables.data_ptr(),
                      tables.shape[1], _ptr(token_list), batch.seq_of_token.data_ptr(),
                      batch.positions.data_ptr(), n, kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim,
-                     float(scale), int(window), int(keep), mod[0], mod[1], mod[2], _stream())
+                     float(scale), int(window), int(aligned), int(keep), mod[0], mod[1], mod[2], *head_out, _stream())
 
     # The decode kernel runs in workgroups of 12 waves from this many (token, KV head) pairs on, or over
     # contexts longer than this; below both, in workgroups of 4 (measured with 32 query heads over 8 KV
@@ -591,7 +620,8 @@ class HipKernels:
 
     def attention_decode(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
                          scale, window, group, token_list=None, n_listed=None, max_ctx=None,
-                         chunk=None, waves=None, mod=(0.0, None, None), keep: int = 0) -> None:
+                         chunk=None, waves=None, mod=(0.0, None, None), keep: int = 0, aligned: bool = False,
+                         head_out=(None, None, 0)) -> None:
         tables = self._check_attention(q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads,
                                        head_dim, group)
         if q.dtype != torch.bfloat16:
@@ -617,13 +647,14 @@ class HipKernels:
         library.call("ra_attention_decode_mod", q.data_ptr(), q_stride, out.data_ptr(), out.stride(0),
                      kcache.data_ptr(), vcache.data_ptr(), tables.data_ptr(), tables.shape[1],
                      _ptr(token_list), None if one_each else batch.seq_of_token.data_ptr(), batch.positions.data_ptr(), n,
-                     kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim, float(scale), int(window), int(keep),
-                     int(chunk), int(max_chunks), int(waves), _ptr(part_o), _ptr(part_ml), mod[0], mod[1], mod[2],
-                     _stream())
+                     kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim, float(scale), int(window), int(aligned),
+                     int(keep), int(chunk), int(max_chunks), int(waves), _ptr(part_o), _ptr(part_ml), mod[0], mod[1], mod[2],
+                     *head_out, _stream())
 
     def attention_prefill(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
                           scale, window, group, tiles, n_tiles, ranges=None, merge=None, n_merge: int = 0,
-                          n_slots: int = 0, mod=(0.0, None, None), keep: int = 0) -> None:
+                          n_slots: int = 0, mod=(0.0, None, None), keep: int = 0, aligned: bool = False,
+                          head_out=(None, None, 0)) -> None:
         """``tiles``: four ints a listed query tile (request row, first token row, queries, first
         position). With ``ranges`` (three ints a listed tile: first key, one past the last, the part's
         slot or -1) some tiles are listed in several parts by keys, and ``merge`` (four ints a cut tile:
@@ -647,12 +678,13 @@ class HipKernels:
                          kcache.data_ptr(), vcache.data_ptr(), tables.data_ptr(), tables.shape[1],
                          tiles.data_ptr(), int(n_tiles), ranges.data_ptr(), merge.data_ptr(), int(n_merge),
                          part_o.data_ptr(), part_ml.data_ptr(), kcache.shape[2] * 16, num_heads, num_kv_heads,
-                         head_dim, float(scale), int(window), int(keep), mod[0], mod[1], mod[2], _stream())
+                         head_dim, float(scale), int(window), int(aligned), int(keep), mod[0], mod[1], mod[2], *head_out,
+                         _stream())
             return
         library.call("ra_attention_prefill_mod", q.data_ptr(), q_stride, out.data_ptr(), out.stride(0),
                      kcache.data_ptr(), vcache.data_ptr(), tables.data_ptr(), tables.shape[1],
                      tiles.data_ptr(), int(n_tiles), kcache.shape[2] * 16, num_heads, num_kv_heads, head_dim,
-                     float(scale), int(window), int(keep), mod[0], mod[1], mod[2], _stream())
+                     float(scale), int(window), int(aligned), int(keep), mod[0], mod[1], mod[2], *head_out, _stream())
 
     # ---------------------------------------------------------------- linear
     def linear(self, x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor,
@@ -985,13 +1017,14 @@ class HipKernels:
     def latent_prep(self, proj: torch.Tensor, q_off: int, dkv_off: int, c_weight: torch.Tensor, eps: float,
                     positions: torch.Tensor, inv_freq: torch.Tensor, rot_dims: int, rot_width: int, rank: int,
                     num_heads: int, head_dim: int, q_lat: torch.Tensor, slots: torch.Tensor,
-                    kcache: torch.Tensor, vcache: torch.Tensor) -> None:
+                    kcache: torch.Tensor, vcache: torch.Tensor, rope_style: int = 0, amp: float = 1.0) -> None:
         """Norm of the latent, rotation of the shared key part and of the queries' rotated parts, cache write.
 
         ``proj`` [T, *] holds the query heads ([head_dim | rot_width] each) from column ``q_off`` and
         [latent (rank) | key part (rot_width)] from ``dkv_off``. The cache row of a token,
         [rms(latent) * c_weight | rotated key part | zeros], goes to ``kcache`` / ``vcache`` (one KV head of
-        size Dp = q_lat.shape[2]) at ``slots``; ``q_lat`` [T, heads, Dp] gets its columns from ``rank`` on."""
+        size Dp = q_lat.shape[2]) at ``slots``; ``q_lat`` [T, heads, Dp] gets its columns from ``rank`` on. Pairs are half-split
+        (``rope_style`` 0) or neighbours (1); sine and cosine are multiplied by ``amp``."""
         _dev(proj, c_weight, positions, inv_freq, q_lat, slots, kcache, vcache)
         T = proj.shape[0]
         if proj.dim() != 2 or proj.stride(1) != 1:
@@ -1010,7 +1043,7 @@ class HipKernels:
             raise ValueError("latent_prep: inv_freq is float32 with rot_dims/2 entries")
         library.call("ra_latent_prep", proj.data_ptr(), _tag(proj, "latent_prep"), proj.stride(0), int(q_off),
                      int(dkv_off), c_weight.data_ptr(), _tag(c_weight, "latent norm weight"), float(eps),
-                     positions.data_ptr(), inv_freq.data_ptr(), int(rot_dims), int(rot_width), int(rank),
+                     positions.data_ptr(), inv_freq.data_ptr(), int(rot_dims), int(rope_style), float(amp), int(rot_width), int(rank),
                      int(num_heads), int(head_dim), q_lat.data_ptr(), Dp, slots.data_ptr(), kcache.data_ptr(),
                      vcache.data_ptr(), kcache.shape[2] * 16, T, _stream())
 

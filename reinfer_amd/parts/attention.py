@@ -25,8 +25,12 @@ rotation, and a head's result is turned back by the query's position), ``out_gat
 sigmoid(W_g h), tensor ``g``) and ``kv_shared`` (no key and value tensors: the layer reads another layer's cache
 with queries of its own), ``values_are_keys`` (no value tensor: a value is the key as projected, before its norm and
 rotation; the product makes q and k alone and the head kernel caches k in both places), ``keep_first`` (with a window: a
-request's first tokens stay in sight, and their blocks stay with the request) and ``out_bias`` (a bias on the output
-projection). With a head norm and heads that are padded with zeros the norm's mean is taken over
+request's first tokens stay in sight, and their blocks stay with the request), ``out_bias`` (a bias on the output
+projection), ``chunked`` (a query sees the keys of its own chunk of ``window``, counted from position 0), ``sink`` (one more
+term exp(s_h) in the softmax's denominator, tensor ``sink`` with one number a query head), ``head_gate`` (a head's result
+times sigmoid(W_g h)_h, tensor ``g`` with a row a query head; its rows ride on the q/k/v product and the attention kernels
+apply it) and ``qk_norm`` without weights (``qk_norm_weights`` False). A layer all of whose options live inside the product,
+the head kernel and the attention kernels (``fused``) takes and hands on the norms around it like plain attention. With a head norm and heads that are padded with zeros the norm's mean is taken over
 the true size: the kernel's mean over D entries with eps * size / D inside the root, times sqrt(size / D) folded
 into the weight, is the same number.
 """
@@ -69,7 +73,14 @@ class GroupedQueryAttention:
     @staticmethod
     def _extended(spec: MixerSpec) -> bool:
         return bool(spec.qk_norm_whole or spec.softcap or spec.distance_bias or spec.rotate_values or spec.out_gate
-                    or spec.kv_shared or spec.values_are_keys or spec.keep_first or spec.out_bias)
+                    or spec.kv_shared or spec.values_are_keys or spec.keep_first or spec.out_bias or spec.chunked
+                    or spec.sink or spec.head_gate or (spec.qk_norm and not spec.qk_norm_weights))
+
+    @staticmethod
+    def _fused(spec: MixerSpec) -> bool:
+        """Whether no further option needs a kernel of its own behind the product or behind the attention."""
+        return not (spec.qk_norm_whole or spec.rotate_values or spec.out_gate or spec.out_bias or spec.bias
+                    or spec.values_are_keys)
 
     @classmethod
     def declare_params(cls, spec: MixerSpec, prefix: str) -> List[ParamDecl]:
@@ -93,7 +104,7 @@ class GroupedQueryAttention:
                     out.append(ParamDecl(prefix + bv, (spec.num_kv_heads * vd,), init="zeros", role=MATRIX))
         if spec.out_bias:
             out.append(ParamDecl(prefix + o + spec.option("bias_suffix", ".bias"), (spec.hidden,), init="zeros", role=MATRIX))
-        if spec.qk_norm or spec.qk_norm_whole:
+        if (spec.qk_norm and spec.qk_norm_weights) or spec.qk_norm_whole:
             nq_name, nk_name = cls._norm_names(spec)
             out.append(ParamDecl(prefix + nq_name, (nq if spec.qk_norm_whole else spec.head_dim,), init="norm", role=VECTOR))
             if own_kv:
@@ -104,6 +115,10 @@ class GroupedQueryAttention:
                     ParamDecl(prefix + "r2", (spec.num_heads,), init="norm", role=VECTOR)]
         if spec.out_gate:
             out.append(ParamDecl(prefix + "g", (spec.num_heads * vd, spec.hidden)))
+        if spec.head_gate:
+            out.append(ParamDecl(prefix + "g", (spec.num_heads, spec.hidden)))
+        if spec.sink:
+            out.append(ParamDecl(prefix + "sink", (spec.num_heads,), role=VECTOR))
         return out
 
     def __init__(self, spec: MixerSpec, weights: Dict[str, torch.Tensor], prefix: str,
@@ -129,7 +144,8 @@ class GroupedQueryAttention:
             raise ValueError("attention: values that are the keys as projected have the keys' size and neither a norm over "
                              "the whole projection, nor a turn of their own, nor another layer's cache beside them")
         self.extended = self._extended(spec)
-        if self.extended:
+        self.fused = self.extended and self._fused(spec)
+        if self.extended and not self.fused:
             # the further options run as kernels of their own around the attention: no norm rides on this
             # mixer's products, and its result goes back to the caller
             self.adds_in_place = self.takes_row_scaled = self.emits_for_norm = False
@@ -139,6 +155,10 @@ class GroupedQueryAttention:
                              "sizes go in steps of 16")
         if spec.qk_norm and spec.qk_norm_whole:
             raise ValueError("attention: q and k are normed per head or over their whole projection, not both")
+        if spec.out_gate and spec.head_gate:
+            raise ValueError("attention: the gate is one number a head or one a value entry, not both")
+        if spec.chunked and (not spec.window or spec.keep_first):
+            raise ValueError("attention: chunks have a size and keep no first tokens")
 
         def heads_of(w, n, d):           # [n * d, ...] -> [n * D, ...], zeros behind each head
             if d == D:
@@ -152,6 +172,15 @@ class GroupedQueryAttention:
             rows.append(heads_of(weights[prefix + kn], G, key_dim))
             if not self.values_are_keys:
                 rows.append(heads_of(weights[prefix + vn], G, value_dim))
+        # columns of the heads in the product's rows; a gate of one number a head stands behind them
+        self.heads_width = sum(int(r.shape[0]) for r in rows)
+        self.gate_cols = 0
+        if spec.head_gate:
+            self.gate_cols = -(-H // 16) * 16
+            gate = weights[prefix + "g"]
+            rows.append(gate)
+            if self.gate_cols > H:
+                rows.append(torch.zeros((self.gate_cols - H, spec.hidden), dtype=gate.dtype, device=gate.device))
         self.w_qkv = torch.cat(rows, dim=0).contiguous()
         self.b_qkv = None
         if spec.bias:
@@ -161,6 +190,8 @@ class GroupedQueryAttention:
                 rows.append(heads_of(weights[prefix + bk], G, key_dim))
                 if not self.values_are_keys:
                     rows.append(heads_of(weights[prefix + bv], G, value_dim))
+            if self.gate_cols:
+                rows.append(torch.zeros(self.gate_cols, dtype=rows[0].dtype, device=rows[0].device))
             self.b_qkv = torch.cat(rows, dim=0).to(dtype).contiguous()
         self.w_o = weights[prefix + on]
         self.b_o = None
@@ -174,8 +205,11 @@ class GroupedQueryAttention:
         self.q_norm = self.k_norm = self.q_whole = self.k_whole = None
         nq_name, nk_name = self._norm_names(spec)
         if spec.qk_norm:
-            self.q_norm = weights[prefix + nq_name]
-            self.k_norm = weights[prefix + nk_name] if self.own_kv else self.q_norm
+            if spec.qk_norm_weights:
+                self.q_norm = weights[prefix + nq_name]
+                self.k_norm = weights[prefix + nk_name] if self.own_kv else self.q_norm
+            else:
+                self.q_norm = self.k_norm = torch.ones(key_dim, dtype=torch.float32, device=self.w_o.device)
             if key_dim != D:
                 # the kernel's mean runs over D entries of which key_dim carry values
                 fold = (key_dim / D) ** 0.5
@@ -193,7 +227,10 @@ class GroupedQueryAttention:
         self.rotation = (self.position.inv_freq, self.position.rotary_dim, self.position.style)
         if self.position.rotary_dim == 0 and self.extended:
             self.rotation = (torch.zeros(D // 2, dtype=torch.float32, device=device), D, 0)
+        if self.position.amplitude != 1.0:
+            raise ValueError("attention: the head kernel turns q and k without a factor on sine and cosine")
         self.softcap = float(spec.softcap)
+        self.sink = weights[prefix + "sink"].float().contiguous() if spec.sink else None
         self.distance = None
         if spec.distance_bias:
             self.distance = (weights[prefix + "r1"].float().contiguous(), weights[prefix + "r2"].float().contiguous())
@@ -209,7 +246,7 @@ class GroupedQueryAttention:
             self.w_gate = heads_of(weights[prefix + "g"], H, value_dim).contiguous()
 
     def cache_need(self) -> KVNeed:
-        return KVNeed(self.num_kv_heads, self.head_dim, self.window, self.keep)
+        return KVNeed(self.num_kv_heads, self.head_dim, self.window, self.keep, bool(self.spec.chunked))
 
     def plan_captured_step(self, batch, num_rows: int, ctx_cap: int) -> None:
         # the attention kernels pick their grids by host-side numbers of the step: the kernel set fixes them
@@ -217,26 +254,22 @@ class GroupedQueryAttention:
         if hook is not None:
             hook(batch, num_rows, ctx_cap)
 
-    def _forward_extended(self, x, batch, cache: LayerCache):
-        """The mixer with any of its further options; the result is float (it enters a float sum as it is)."""
+    def _forward_extended(self, x, batch, cache: LayerCache, resid=None, emit: Optional[NormTarget] = None):
+        """The mixer with any of its further options. Where they live inside the kernels of plain attention (``fused``) its
+        result goes the same way; else it is float (it enters a float sum as it is)."""
         ops = kernels.current()
+        x, row_sums = split_input(x)
         T = x.shape[0]
         H, G, D = self.num_heads, self.num_kv_heads, self.head_dim
-        # a layer without keys of its own makes queries alone; where the head kernel must still run over them (a
-        # head norm, a rotation) the key and value parts it expects are zeros that nothing stores
+        # a layer without keys of its own makes queries alone; the head kernel still runs over them where they are
+        # normed or turned
         head_kernel = self.own_kv or self.q_norm is not None or self.position.rotary_dim > 0
-        width = (H + (1 if self.values_are_keys else 2) * G) * D if head_kernel else H * D
-        if self.own_kv:
-            qkv = torch.empty((T, width), dtype=self.dtype, device=x.device)
+        width = self.heads_width + self.gate_cols
+        qkv = torch.empty((T, width), dtype=self.dtype, device=x.device)
+        if row_sums is None:
             ops.linear(x, self.w_qkv, qkv, self.b_qkv)
-        elif head_kernel:
-            qkv = torch.zeros((T, width), dtype=self.dtype, device=x.device)
-            q_only = torch.empty((T, H * D), dtype=self.dtype, device=x.device)
-            ops.linear(x, self.w_qkv, q_only, self.b_qkv)
-            qkv[:, :H * D] = q_only
         else:
-            qkv = torch.empty((T, width), dtype=self.dtype, device=x.device)
-            ops.linear(x, self.w_qkv, qkv, self.b_qkv)
+            ops.linear_skinny(x, self.w_qkv, qkv, self.b_qkv, row_sums=row_sums)
         if self.q_whole is not None:
             spans = [(0, H * D, self.q_whole, H * self.key_dim)]
             if self.own_kv:
@@ -250,10 +283,12 @@ class GroupedQueryAttention:
             inv_freq, rotary_dim, style = self.rotation
             more = {"values_are_keys": True} if self.values_are_keys else {}
             ops.qk_norm_rope_cache(qkv, self.q_norm, self.k_norm, self.eps, batch.positions, inv_freq, rotary_dim, style,
-                                   slots, cache.k, cache.v, H, G, D, **more)
+                                   slots, cache.k, cache.v, H, G if self.own_kv else 0, D, **more)
         attn = torch.empty((T, H * D), dtype=self.dtype, device=x.device)
         ops.attention(qkv, width, attn, cache.k, cache.v, batch, H, G, D, self.scale, self.window, cache.group,
-                      softcap=self.softcap, distance=self.distance, **({"keep": self.keep} if self.keep else {}))
+                      softcap=self.softcap, distance=self.distance, **self._call_options(qkv))
+        if self.fused:
+            return self._project_out(ops, attn, resid, emit)
         if self.value_inv_freq is not None or self.w_gate is not None:
             gate = None
             if self.w_gate is not None:
@@ -266,10 +301,23 @@ class GroupedQueryAttention:
         ops.linear(attn, self.w_o, out, self.b_o)
         return out
 
+    def _call_options(self, qkv):
+        """What the attention call is handed beside the options every extended layer names."""
+        more = {}
+        if self.keep:
+            more["keep"] = self.keep
+        if self.spec.chunked:
+            more["aligned"] = True
+        if self.sink is not None:
+            more["sink"] = self.sink
+        if self.gate_cols:
+            more["gate"] = qkv[:, self.heads_width:]
+        return more
+
     def forward(self, x, batch, cache: LayerCache, resid: Optional[torch.Tensor] = None,
                 emit: Optional[NormTarget] = None):
         if self.extended:
-            return self._forward_extended(split_input(x)[0], batch, cache)
+            return self._forward_extended(x, batch, cache, resid, emit)
         ops = kernels.current()
         x, row_sums = split_input(x)
         T = x.shape[0]
@@ -297,6 +345,10 @@ class GroupedQueryAttention:
         attn = torch.empty((T, self.num_heads * self.head_dim), dtype=self.dtype, device=x.device)
         ops.attention(q_rows, q_stride, attn, cache.k, cache.v, batch, self.num_heads,
                       self.num_kv_heads, self.head_dim, self.scale, self.window, cache.group)
+        return self._project_out(ops, attn, resid, emit)
+
+    def _project_out(self, ops, attn, resid, emit: Optional[NormTarget]):
+        T = attn.shape[0]
         can_add = getattr(ops, "can_accumulate", None)
         if resid is not None and can_add and can_add(attn, self.w_o):
             # x += attn . Wo^T in the epilogue, which can also prepare the norm that follows
@@ -309,6 +361,6 @@ class GroupedQueryAttention:
                 return emit
             ops.linear_skinny(attn, self.w_o, resid, accumulate=True)
             return None
-        out = torch.empty((T, self.spec.hidden), dtype=self.dtype, device=x.device)
+        out = torch.empty((T, self.spec.hidden), dtype=self.dtype, device=attn.device)
         ops.linear(attn, self.w_o, out)
         return out

@@ -1,7 +1,7 @@
 """What a mixer asks of the cache, and what a layer is handed at run time."""
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Optional, Tuple
 
 import torch
@@ -15,10 +15,12 @@ class PagedNeed:
     engine allocates ``[blocks, *shape]`` for each and hands them over in ``LayerCache.tensors`` by name;
     token slot s of the step (``batch.slots[group]``) is slot ``s % block_size`` of block ``s // block_size``,
     wherever in its block's shape the mixer puts it. ``window`` W > 0: only the last W tokens are read, the
-    blocks behind them go back to the pool, but for those that hold the request's first ``keep`` tokens."""
+    blocks behind them go back to the pool, but for those that hold the request's first ``keep`` tokens.
+    ``chunked``: read are the tokens of the same chunk of W, counted from position 0; the chunks behind go back."""
     tensors: Tuple[Tuple[str, Tuple[int, ...], Optional[torch.dtype]], ...]
     window: int = 0
     keep: int = 0
+    chunked: bool = False
 
     def block_tensors(self, block_size: int):
         return tuple((name, tuple(block_size if n == -1 else n for n in shape), dtype)
@@ -34,6 +36,7 @@ class KVNeed:
     head_dim: int
     window: int = 0
     keep: int = 0           # first tokens that a window keeps in sight
+    chunked: bool = False   # the window is the query's own chunk of that many tokens, counted from position 0
 
     def block_tensors(self, block_size: int):
         from ..cache.layout import cache_shape
@@ -61,6 +64,19 @@ class JointNeed:
         if len(found) > 1:
             raise ValueError("a layer's mixers may keep pages in one of them only")
         return found[0] if found else None
+
+
+def covering(need, other):
+    """``need`` with a window that also covers what a layer of need ``other`` reads of the same pages: the wider of
+    two windows; of two chunk sizes the larger if it is a multiple of the smaller, else (and for a chunk beside a window: no
+    chunk reaches further back than its size) a sliding window of the larger; everything where either reads everything."""
+    a, b = (need.window, need.chunked), (other.window, other.chunked)
+    keep = max(need.keep, other.keep)
+    if not a[0] or not b[0]:
+        return replace(need, window=0, keep=0, chunked=False)
+    wide, narrow = max(a[0], b[0]), min(a[0], b[0])
+    chunked = a[1] and b[1] and wide % narrow == 0 and not keep
+    return replace(need, window=wide, keep=keep, chunked=chunked)
 
 
 def paged_need(need):

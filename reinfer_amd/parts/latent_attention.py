@@ -19,6 +19,8 @@ q, the latent and the gate come from one fused product.
 Two options. ``q_rank`` > 0: the queries come through a latent of their own, q = W_uq (rms(W_dq h) * w_q): the
 fused product then makes [latent of q | latent | key part | gate], a row norm and a second product make q.
 ``head_gate``: the gate is one number a head, sigmoid(W_g h)_a with W_g [heads, width], not one a value entry.
+The rotation turns half-split pairs or neighbours (the position part's ``style``), its sine and cosine times the part's
+``amplitude``.
 """
 from __future__ import annotations
 
@@ -121,6 +123,7 @@ class LatentAttention:
         self.w_values = weights[prefix + "uv"].view(H, Dv, self.rank).contiguous()
         self.w_o = weights[prefix + "o"]
         self.position = lookup("position", spec.position.kind)(spec.position, device)
+        self.turned_otherwise = self.position.style != 0 or self.position.amplitude != 1.0
         if self.position.rotary_dim > R:
             raise ValueError("the rotated width cannot exceed the rotated part of a head")
 
@@ -170,7 +173,8 @@ class LatentAttention:
         q_lat = torch.empty((T, H, Dp), dtype=self.dtype, device=x.device)
         ops.latent_prep(proj, self.q_off, self.dkv_off, self.c_norm, self.eps, batch.positions,
                         self.position.inv_freq, self.position.rotary_dim, self.rot_width, self.rank, H, D,
-                        q_lat, slots, cache.k, cache.v)
+                        q_lat, slots, cache.k, cache.v,
+                        **({"rope_style": self.position.style, "amp": self.position.amplitude} if self.turned_otherwise else {}))
         q_rows = q_lat.view(T, H * Dp)
         if D > 0:
             ops.head_linear(proj[:, self.q_off:], D + self.rot_width, self.w_absorb, q_rows, Dp)

@@ -48,7 +48,8 @@ class KernelDouble:
                            rope_style, slots, kcache, vcache, num_heads, num_kv_heads, head_dim, values_are_keys=False):
         T = qkv.shape[0]
         d = head_dim
-        u = qkv.view(T, num_heads + (1 if values_are_keys else 2) * num_kv_heads, d).float()
+        n = num_heads + (1 if values_are_keys else 2) * num_kv_heads
+        u = qkv[:, :n * d].reshape(T, n, d).float()
         q, k = u[:, :num_heads], u[:, num_heads:num_heads + num_kv_heads]
         v = k if values_are_keys else u[:, num_heads + num_kv_heads:]
 
@@ -76,7 +77,9 @@ class KernelDouble:
 
         q = rot(norm(q, q_weight))
         k = rot(norm(k, k_weight))
-        qkv.view(T, -1, d)[:, :num_heads] = q.to(qkv.dtype)
+        qkv[:, :num_heads * d] = q.reshape(T, -1).to(qkv.dtype).clone()
+        if num_kv_heads == 0:
+            return
         bs = kcache.shape[2] * 16
         kflat, vflat = kcache.view(kcache.shape[0], num_kv_heads, -1), vcache.view(vcache.shape[0], num_kv_heads, -1)
         e = torch.arange(d)
@@ -118,7 +121,7 @@ class KernelDouble:
 
     # ---- latent attention
     def latent_prep(self, proj, q_off, dkv_off, c_weight, eps, positions, inv_freq, rot_dims, rot_width, rank,
-                    num_heads, head_dim, q_lat, slots, kcache, vcache):
+                    num_heads, head_dim, q_lat, slots, kcache, vcache, rope_style=0, amp=1.0):
         T = proj.shape[0]
         Dp = q_lat.shape[2]
         half = rot_dims // 2
@@ -128,8 +131,13 @@ class KernelDouble:
             if not half:
                 return x
             shape = [T] + [1] * (x.dim() - 2) + [half]
-            c, s = torch.cos(ang).view(shape), torch.sin(ang).view(shape)
+            c, s = amp * torch.cos(ang).view(shape), amp * torch.sin(ang).view(shape)
             out = x.clone()
+            if rope_style == 1:
+                a, b = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
+                out[..., 0:rot_dims:2] = a * c - b * s
+                out[..., 1:rot_dims:2] = b * c + a * s
+                return out
             a, b = x[..., :half], x[..., half:rot_dims]
             out[..., :half] = a * c - b * s
             out[..., half:rot_dims] = b * c + a * s
@@ -594,7 +602,7 @@ class KernelDouble:
                 so[p] = sq[:, p * part:(p + 1) * part].sum(1)
 
     def attention(self, q, q_stride, out, kcache, vcache, batch, num_heads, num_kv_heads, head_dim,
-                  scale, window, group, softcap=0.0, distance=None, keep=0):
+                  scale, window, group, softcap=0.0, distance=None, keep=0, aligned=False, sink=None, gate=None):
         T = batch.num_tokens
         bs = kcache.shape[2] * 16
         kl, vl = unpack_k(kcache, head_dim), unpack_v(vcache, head_dim)      # [blocks, Hkv, bs, d]
@@ -605,6 +613,8 @@ class KernelDouble:
             seq = int(batch.seq_of_token[t])
             p = int(batch.positions[t])
             lo = max(0, p - window + 1) if window > 0 else 0
+            if aligned and window > 0:
+                lo = p // window * window
             keys = torch.cat([torch.arange(0, min(keep, lo)), torch.arange(lo, p + 1)])
             blk = tables[seq, keys // bs].long()
             K = kl[blk, :, keys % bs, :].float()        # [n, Hkv, d]
@@ -615,8 +625,13 @@ class KernelDouble:
                     s = softcap * torch.tanh(s / softcap)
                 if distance is not None:
                     s = s - distance[0][a] * torch.log(1.0 + distance[1][a] * (p - keys).float())
-                pr = torch.softmax(s, dim=0)
-                out[t, a * head_dim:(a + 1) * head_dim] = (pr @ V[:, a // ratio, :]).to(out.dtype)
+                if sink is not None:                # a last score without a value
+                    s = torch.cat([s, sink[a:a + 1]])
+                pr = torch.softmax(s, dim=0)[:keys.numel()]
+                o = pr @ V[:, a // ratio, :]
+                if gate is not None:
+                    o = o * torch.sigmoid(gate[t, a].float())
+                out[t, a * head_dim:(a + 1) * head_dim] = o.to(out.dtype)
 
     attention_plain = attention
 
