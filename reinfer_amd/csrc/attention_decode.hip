@@ -78,7 +78,9 @@ __device__ __forceinline__ int fd_kept(int keep, int lo) {
 // FLAGS & FD_MOD: the scores are changed before the softmax (RaScoreMod: a tanh cap, a per-head distance term)
 // FLAGS & FD_KEEP: a window that keeps the first keys. The walk is over one run of places: from the window's first
 // tile on a place is the key's own number, and the kept tiles take the places right below it.
-enum { FD_MOD = 1, FD_KEEP = 2 };
+// FLAGS & FD_HEAD: the window may be the query's own chunk (aligned), and the head's result has a sink and / or a gate
+// (RaHeadOut); the other forms keep their scalar registers.
+enum { FD_MOD = 1, FD_KEEP = 2, FD_HEAD = 4 };
 template <int DMAX, bool EXACT, int FD_WAVES, int FLAGS>
 __global__ void __launch_bounds__(FD_WAVES * RA_WAVE, (DMAX <= 128 && FD_WAVES == 4) ? 3 : 1)
 flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
@@ -89,7 +91,7 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
                     float scale_log2, int window, int keep, int chunk_shift, int max_chunks, int n_tokens,
                     int t_base, float* __restrict__ part_o, float* __restrict__ part_ml, float scale, RaScoreMod mod,
                     int aligned, RaHeadOut ho) {
-  constexpr bool MOD = (FLAGS & FD_MOD) != 0, KEEP = (FLAGS & FD_KEEP) != 0;
+  constexpr bool MOD = (FLAGS & FD_MOD) != 0, KEEP = (FLAGS & FD_KEEP) != 0, HEAD = (FLAGS & FD_HEAD) != 0;
   constexpr int FD_THREADS = FD_WAVES * RA_WAVE;
   const int d = EXACT ? DMAX : d_arg;
   constexpr int NDT = DMAX / 32;       // 32-wide d tiles of the score product
@@ -111,7 +113,7 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
     // seq_of_token null: every request of the step brings one token, token t is request t
     const int seq = seq_of_token ? seq_of_token[t] : t;
     const int p = positions[t];
-    const int lo = ra_first_key(p, window, aligned);
+    const int lo = ra_first_key(p, window, HEAD ? aligned : 0);
     const int keep16 = KEEP ? fd_kept(keep, lo) : 0;
     const FdCut cut = fd_cut(p, lo, keep16, chunk_shift, max_chunks, FD_WAVES * 32);
     const int n_chunks = cut.n;
@@ -288,8 +290,11 @@ flash_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restri
       }
       if (n_chunks == 1) {
         const int head = kvh * G + h;
-        lt += ra_sink_term(ho, head, mw);
-        out[(size_t)t * out_stride + (size_t)head * d + e] = from_f32<bf16_t>(ot / lt * ra_head_gate<bf16_t>(ho, t, head));
+        if (HEAD) {
+          lt += ra_sink_term(ho, head, mw);
+          ot *= ra_head_gate<bf16_t>(ho, t, head);
+        }
+        out[(size_t)t * out_stride + (size_t)head * d + e] = from_f32<bf16_t>(ot / lt);
       } else {
         part_o[(prow + h) * d + e] = ot;
         if (e == 0) {
@@ -432,9 +437,10 @@ static size_t fd_lds_limit(void) {
 template <int DM, bool EX, int WV>
 static hipError_t fd_allow_lds(size_t lds) {
   if (lds <= 64 * 1024) return hipSuccess;
-  const void* forms[4] = {(const void*)flash_decode_kernel<DM, EX, WV, 0>, (const void*)flash_decode_kernel<DM, EX, WV, FD_MOD>,
-                          (const void*)flash_decode_kernel<DM, EX, WV, FD_KEEP>,
-                          (const void*)flash_decode_kernel<DM, EX, WV, FD_MOD | FD_KEEP>};
+  const void* forms[8] = {(const void*)flash_decode_kernel<DM, EX, WV, 0>, (const void*)flash_decode_kernel<DM, EX, WV, 1>,
+                          (const void*)flash_decode_kernel<DM, EX, WV, 2>, (const void*)flash_decode_kernel<DM, EX, WV, 3>,
+                          (const void*)flash_decode_kernel<DM, EX, WV, 4>, (const void*)flash_decode_kernel<DM, EX, WV, 5>,
+                          (const void*)flash_decode_kernel<DM, EX, WV, 6>, (const void*)flash_decode_kernel<DM, EX, WV, 7>};
   for (const void* f : forms) {
     const hipError_t e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
@@ -518,6 +524,7 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
   const RaScoreMod mod = {softcap, r1, r2};
   const RaHeadOut ho = {sink, gate, gate_stride};
   const bool changed = softcap > 0.f || r1 != nullptr;
+  const bool head = aligned || sink != nullptr || gate != nullptr;
   RA_CHECK(n_tokens > 0, "attention_decode: no tokens");
   RA_CHECK(ra_attention_decode_supports(Hq, Hkv, d, block_size),
            "attention_decode: unsupported sizes (%d query heads, %d KV heads, head size %d, block %d)", Hq,
@@ -548,14 +555,22 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
   (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache, (const bf16_t*)vcache, \
       block_tables, max_blocks, token_list, seq_of_token, positions, block_size, Hkv, G, d, scale_log2, \
       window, keep, chunk_shift, max_chunks, n_tokens, 0, part_o, part_ml, scale, mod, aligned, ho
+#define RA_FD_FORM(DM, EX, WV, F) \
+  case F: flash_decode_kernel<DM, EX, WV, F><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); break;
 #define RA_FD_GO(DM, EX, WV)                                                                          \
   do {                                                                                                \
     if (fd_allow_lds<DM, EX, WV>(lds) != hipSuccess)                                                  \
       return ra_fail("attention_decode: the device does not give a workgroup %zu bytes of LDS", lds); \
-    if (changed && keep > 0) flash_decode_kernel<DM, EX, WV, FD_MOD | FD_KEEP><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); \
-    else if (changed) flash_decode_kernel<DM, EX, WV, FD_MOD><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); \
-    else if (keep > 0) flash_decode_kernel<DM, EX, WV, FD_KEEP><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS); \
-    else flash_decode_kernel<DM, EX, WV, 0><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS);         \
+    switch ((changed ? FD_MOD : 0) | (keep > 0 ? FD_KEEP : 0) | (head ? FD_HEAD : 0)) {               \
+      RA_FD_FORM(DM, EX, WV, 1)                                                                       \
+      RA_FD_FORM(DM, EX, WV, 2)                                                                       \
+      RA_FD_FORM(DM, EX, WV, 3)                                                                       \
+      RA_FD_FORM(DM, EX, WV, 4)                                                                       \
+      RA_FD_FORM(DM, EX, WV, 5)                                                                       \
+      RA_FD_FORM(DM, EX, WV, 6)                                                                       \
+      RA_FD_FORM(DM, EX, WV, 7)                                                                       \
+      default: flash_decode_kernel<DM, EX, WV, 0><<<grid, WV * RA_WAVE, lds, stream>>>(RA_FD_ARGS);   \
+    }                                                                                                 \
   } while (0)
 #define RA_FD(DM)                                                                                     \
   do {                                                                                                \
@@ -571,6 +586,7 @@ extern "C" int ra_attention_decode_mod(const void* q, int q_stride, void* out, i
   else if (d <= 128) RA_FD(128);
   else RA_FD(256);
 #undef RA_FD_GO
+#undef RA_FD_FORM
 #undef RA_FD
 #undef RA_FD_ARGS
   RA_LAUNCH_CHECK("attention_decode");

@@ -227,7 +227,7 @@ class GroupedQueryAttention:
         self.rotation = (self.position.inv_freq, self.position.rotary_dim, self.position.style)
         if self.position.rotary_dim == 0 and self.extended:
             self.rotation = (torch.zeros(D // 2, dtype=torch.float32, device=device), D, 0)
-        if self.position.amplitude != 1.0:
+        if getattr(self.position, "amplitude", 1.0) != 1.0:
             raise ValueError("attention: the head kernel turns q and k without a factor on sine and cosine")
         self.softcap = float(spec.softcap)
         self.sink = weights[prefix + "sink"].float().contiguous() if spec.sink else None

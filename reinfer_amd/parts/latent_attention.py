@@ -123,7 +123,8 @@ class LatentAttention:
         self.w_values = weights[prefix + "uv"].view(H, Dv, self.rank).contiguous()
         self.w_o = weights[prefix + "o"]
         self.position = lookup("position", spec.position.kind)(spec.position, device)
-        self.turned_otherwise = self.position.style != 0 or self.position.amplitude != 1.0
+        self.amplitude = float(getattr(self.position, "amplitude", 1.0))
+        self.turned_otherwise = self.position.style != 0 or self.amplitude != 1.0
         if self.position.rotary_dim > R:
             raise ValueError("the rotated width cannot exceed the rotated part of a head")
 
@@ -174,7 +175,7 @@ class LatentAttention:
         ops.latent_prep(proj, self.q_off, self.dkv_off, self.c_norm, self.eps, batch.positions,
                         self.position.inv_freq, self.position.rotary_dim, self.rot_width, self.rank, H, D,
                         q_lat, slots, cache.k, cache.v,
-                        **({"rope_style": self.position.style, "amp": self.position.amplitude} if self.turned_otherwise else {}))
+                        **({"rope_style": self.position.style, "amp": self.amplitude} if self.turned_otherwise else {}))
         q_rows = q_lat.view(T, H * Dp)
         if D > 0:
             ops.head_linear(proj[:, self.q_off:], D + self.rot_width, self.w_absorb, q_rows, Dp)

@@ -51,6 +51,35 @@ def test_plan_groups_tells_windows_that_keep_first_tokens_apart():
     assert [(g.window, g.keep, g.entries) for g in groups] == [(0, 0, (3,)), (4, 0, (5,)), (8, 0, (0,)), (8, 3, (1, 4))]
 
 
+def test_plan_groups_tells_chunks_and_windows_apart():
+    groups = plan_groups([8, 8, 0, 8, None], None, [True, False, True, True, False])
+    assert [(g.window, g.chunked, g.entries) for g in groups] == [(0, False, (2,)), (8, False, (1,)), (8, True, (0, 3))]
+
+
+def test_chunks_are_given_back_whole_when_the_next_one_begins():
+    """Blocks of four tokens, chunks of ten: a block stays while any later query's chunk holds a token of it; a portion over
+    several chunks needs the blocks from its first query's chunk on."""
+    m = CacheManager([CacheGroupSpec(window=10, entries=(0,), chunked=True)], 4, [8], 2)
+    m.add("a")
+    for total in range(1, 41):
+        m.grow("a", total)
+        m.commit("a", total)
+        table = m.get("a").tables[0]
+        first = total // 10 * 10 // 4                      # the next query's chunk begins in this block
+        assert [b >= 0 for b in table] == [i >= first for i in range(len(table))], total
+        m.check()
+    m.free("a")
+    assert m.pools[0].num_free == 8
+    m.add("b")
+    m.grow("b", 9)
+    m.commit("b", 9)
+    assert m.blocks_needed("b", 30) == [8 - 3] and [b >= 0 for b in m.get("b").tables[0]] == [True] * 3
+    m.grow("b", 30)
+    m.commit("b", 30)                                      # the next query begins a chunk: block 7 holds tokens 28 to 31
+    assert [b >= 0 for b in m.get("b").tables[0]] == [False] * 7 + [True]
+    m.check()
+
+
 def test_a_window_keeps_the_blocks_of_its_first_tokens():
     """Blocks of four tokens, a window of six, five kept tokens: the first two blocks stay with the request, the blocks
     between them and the window go back, and all come back once at the end."""

@@ -6,7 +6,7 @@ from reinfer_amd.kernels.ops import HipKernels
 ROOM = 32
 
 
-def plan(portions, room=ROOM, halves=True, tile=64):
+def plan(portions, room=ROOM, halves=True, tile=64, chunk=0):
     """``portions``: (tokens, tokens already cached) of each request of a step."""
     ops = HipKernels.__new__(HipKernels)         # the choice needs no loaded library
     tiles, row = [], 0
@@ -14,7 +14,7 @@ def plan(portions, room=ROOM, halves=True, tile=64):
         for q0 in range(0, n, tile):
             tiles.append((i, row + q0, min(tile, n - q0), start + q0))
         row += n
-    return tiles, ops._prefill_items(tiles, room, halves)
+    return tiles, ops._prefill_items(tiles, room, halves, chunk=chunk)
 
 
 def covered(tiles, items, merge, n_slots):
@@ -54,6 +54,20 @@ def test_a_whole_prompt_that_fills_the_chip_lists_its_heaviest_tiles_twice_by_he
     assert n_slots == 0 and len(items) == len(tiles) + ROOM // 4
     halved = {it[1][3] for it in items if it[1][2] >> 16}
     assert halved == {pos for (_, _, _, pos) in sorted(tiles, key=lambda t: -t[3])[:ROOM // 4]}
+
+
+def test_chunks_are_priced_by_the_keys_that_their_queries_see():
+    """Layers whose queries see their own chunk alone: a tile deep in the prompt is no heavier than one at its start, and
+    where tiles are cut the parts share the rounds from the chunk's start on, the first part taking whatever lies below."""
+    R = HipKernels.PREFILL_ROUND
+    tiles, (items, merge, n_slots) = plan([(2048, 4096)], chunk=256)
+    covered(tiles, items, merge, n_slots)
+    assert n_slots == 0 and max(it[0] for it in items) <= 256 // R + 1
+    tiles, (items, merge, n_slots) = plan([(128, 7000)], chunk=4096)
+    covered(tiles, items, merge, n_slots)
+    assert n_slots > 0
+    for _, (_, _, _, pos), lo, hi, slot in items:
+        assert slot >= 0 and (lo == 0 or lo > pos // 4096 * 4096), "only a tile's first part begins below its chunk"
 
 
 def test_without_halves_a_whole_prompt_is_listed_as_it_is():

@@ -333,20 +333,16 @@ def test_trace_run_gibavik(tmp_path, which, dtype):
         assert_close(torch.cat(got[r]), refs[r], dtype, r)
 
 
-@pytest.mark.parametrize("which,dtype", [("A", "float32"), ("C", "bfloat16"), ("E", "float32")])
-def test_trace_run_sagalorn(tmp_path, which, dtype):
-    """A design with several residual streams, a repeated run of layers, states in slots and windows that keep the first
-    tokens through the same program: five requests on four state slots and a cache for the 320 tokens that the four live
-    ones hold at most, portions beside single tokens, a request left out of a step, slots and blocks taken again."""
-    import plain_sagalorn
-    import sagalorn_helpers as sh
-    from test_sagalorn_engine import assert_close, moved_by_rounding
-    folder = sh.make_folder(tmp_path, which, dtype)
-    raw, weights = sh.read_folder(folder)
+def replay_five_requests(tmp_path, plain, design, checks, which, dtype):
+    """Five requests on four state slots and a cache for the 320 tokens that the four live ones hold at most, portions beside
+    single tokens, a request left out of a step, slots and blocks taken again; every logit against the plain implementation.
+    ``design``: the module with the design's folders, ``checks`` the one with its bounds."""
+    folder = design.make_folder(tmp_path, which, dtype)
+    raw, weights = design.read_folder(folder)
     V = raw["vocab"]
     lens = {"a": 70, "b": 41, "c": 50, "d": 9, "e": 30}
     seqs = {r: random_tokens(n, V, 10 + i) for i, (r, n) in enumerate(lens.items())}
-    refs = {r: plain_sagalorn.forward(raw, weights, t).float() for r, t in seqs.items()}
+    refs = {r: plain.forward(raw, weights, t).float() for r, t in seqs.items()}
     plan = [[("a", 33), ("b", 2)], [("a", 36), ("c", 17), ("d", 3)], [("b", 38), ("d", 1), ("c", 2)],
             [("a", 1), ("b", 1), ("c", 30), ("d", 5)], [("c", 1), ("e", 29)], [("e", 1)]]
     fed = {r: 0 for r in seqs}
@@ -376,4 +372,23 @@ def test_trace_run_sagalorn(tmp_path, which, dtype):
             o += len(e["want"])
         assert o == rows.shape[0]
     for r in seqs:
-        assert_close(torch.cat(got[r]), refs[r], dtype, r, moved_by_rounding(raw, weights, seqs[r], dtype, refs[r]))
+        checks.assert_close(torch.cat(got[r]), refs[r], dtype, r, checks.moved_by_rounding(raw, weights, seqs[r], dtype, refs[r]))
+
+
+@pytest.mark.parametrize("which,dtype", [("A", "float32"), ("C", "bfloat16"), ("E", "float32")])
+def test_trace_run_sagalorn(tmp_path, which, dtype):
+    """A design with several residual streams, a repeated run of layers, states in slots and windows that keep the first
+    tokens through the same program."""
+    import plain_sagalorn
+    import sagalorn_helpers
+    import test_sagalorn_engine
+    replay_five_requests(tmp_path, plain_sagalorn, sagalorn_helpers, test_sagalorn_engine, which, dtype)
+
+
+@pytest.mark.parametrize("which,dtype", [("A", "float32"), ("C", "bfloat16"), ("E", "bfloat16")])
+def test_trace_run_dokanex(tmp_path, which, dtype):
+    """A design with attention inside chunks, keys of earlier layers and latents through the same program."""
+    import dokanex_helpers
+    import plain_dokanex
+    import test_dokanex_engine
+    replay_five_requests(tmp_path, plain_dokanex, dokanex_helpers, test_dokanex_engine, which, dtype)
