@@ -581,10 +581,62 @@ def sagalorn_sizes():
     return out
 
 
+# ---------------------------------------------------------------------------------------------------
+# --design dokanex: the Dokanex design beside the two others that it is closest to, at equal size: Gibavik (its attention
+# layers, readers of an earlier layer's keys among them) and Detatar (its latent layers)
+# ---------------------------------------------------------------------------------------------------
+def _dokanex_raw(width, vocab, pattern, attn, latent_heads, q_rank, ff):
+    """``pattern``: a string of layer codes: A attention, r attention on the keys of the attention layer before it, L latent
+    attention, each with a dense feed-forward."""
+    full = {"dim": 128, "heads": attn[0], "kv_heads": attn[1], "mask": {"size": 1024}, "scale": 128 ** -0.5, "softcap": 15.0,
+            "vdim": 128}
+    latent = {"dim": 128, "heads": latent_heads, "kv_rank": 192, "q_rank": q_rank, "rot_dim": 64, "scale": 192 ** -0.5,
+              "vdim": 128, "rot": {"base": 500000.0, "dims": 64,
+                                   "scaling": {"factor": 4.0, "fast": 32.0, "original": 8192, "slow": 1.0}}}
+    layers = []
+    for c in pattern:
+        mixer = latent if c == "L" else full
+        if c == "r":
+            mixer = dict(full, kv_from=max(i for i, L in enumerate(layers)
+                                           if L["type"] == "attention" and "kv_from" not in L["mixer"]))
+        layers.append({"type": "latent_attention" if c == "L" else "attention", "mixer": mixer,
+                       "mlp": {"ff": ff, "kind": "dense"}})
+    return {"architecture": "Dokanex", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 8.0},
+            "logit_softcap": 25.0, "layers": layers}
+
+
+# (name, Dokanex configuration, its Gibavik twin, vocabulary, "gibavik", ("detatar", its Detatar twin)): as many layers, the
+# same width and heads; the Gibavik twin has attention layers alone (a window of 1,024 where Dokanex has chunks of 1,024), the
+# Detatar twin latent layers alone; a twin's feed-forward width (a multiple of 64) brings its parameter count closest
+def dokanex_sizes():
+    out = []
+    for name, width, attn, latent_heads, q_rank, ff in (("w2048", 2048, (16, 4), 16, 768, 5632),
+                                                        ("w4096", 4096, (32, 8), 16, 1536, 11008)):
+        vocab, pattern = 32768, "ALrALr"
+        raw = _dokanex_raw(width, vocab, pattern, attn, latent_heads, q_rank, ff)
+
+        def gibavik(tff):
+            g = _gibavik_raw(width, vocab, pattern.replace("L", "A"), attn, 16, tff, (1, 1, 64))
+            for L in g["layers"]:
+                L["mlp"] = {"ff": tff, "kind": "dense", "limit": 7.0}
+                L["mixer"] = dict(L["mixer"], mask={"size": 1024})
+            return g
+
+        def detatar(tff):
+            return _detatar_raw(width, vocab, "A" * len(pattern), latent_heads, 192, q_rank, 32, tff, (16, 4, 64, 64))
+
+        def fitted(twin):
+            want, a, b = _parameters(raw), _parameters(twin(1024)), _parameters(twin(2048))
+            return twin(max(64, round((1024 + (want - a) * 1024 / (b - a)) / 64) * 64))
+        out.append((name, raw, fitted(gibavik), vocab, "gibavik", ("detatar", fitted(detatar))))
+    return out
+
+
 def design_run(args) -> int:
     """Prefill and decode throughput of the design (``--design``) and of its twin at each size, and the GPU time of a
     2,048-token prompt step and of a decode step at batch 8 by kernel class with each class's share of its
-    roofline (weight bytes over 8 TB/s or flops over 2.5 PFLOP/s, whichever is longer). One JSON line."""
+    roofline (bytes of weights, or of keys and values, over 8 TB/s or flops over 2.5 PFLOP/s, whichever is longer). One JSON
+    line."""
     import gc
     import torch
     from reinfer_amd import kernels
@@ -603,7 +655,7 @@ def design_run(args) -> int:
             runner.add_request(r)
             if ctx:
                 runner.step([StepEntry(r, torch.randint(0, vocab, (ctx,), generator=g).tolist(), [])])
-        timed = TimedKernels(kernels.current())
+        timed = TimedKernels(kernels.current(), attention_shapes=True)
         graphs, runner.graphs = runner.graphs, None
         try:
             with kernels.use(timed):
@@ -624,13 +676,14 @@ def design_run(args) -> int:
 
     results = {}
     sizes = {"kobolix": kobolix_sizes, "puresun": design_sizes, "detatar": detatar_sizes,
-             "gibavik": gibavik_sizes, "sagalorn": sagalorn_sizes}[args.design]()
+             "gibavik": gibavik_sizes, "sagalorn": sagalorn_sizes, "dokanex": dokanex_sizes}[args.design]()
     twin_name = "qwen3"
     for name, p_raw, q_raw, vocab, *rest in sizes:
         twin_name = rest[0] if rest else "qwen3"
+        twins = [(twin_name, q_raw), *rest[1:]]
         if args.size and name != args.size:
             continue
-        for which, raw in ((args.design, p_raw), (twin_name, q_raw)):
+        for which, raw in ((args.design, p_raw), *twins):
             cfg = config_from_dict(raw)
             log(f"{name} {which}: building ...")
             engine = LLMEngine(config=cfg, seed=args.seed, dtype=args.dtype, block_size=16,
@@ -683,9 +736,10 @@ def main() -> int:
     ap.add_argument("--max-model-len", type=int, default=None, metavar="N",
                     help="context length (default: the shape's: 4096 at 8b, 8192 at 4b, 16384 at 32b)")
     ap.add_argument("--shape", default="8b", choices=sorted(SHAPES), help="layer sizes (default: the Qwen3-8B shape)")
-    ap.add_argument("--design", default=None, choices=["puresun", "kobolix", "detatar", "gibavik", "sagalorn"],
+    ap.add_argument("--design", default=None, choices=["puresun", "kobolix", "detatar", "gibavik", "sagalorn", "dokanex"],
                     help="instead of the default measurement: this design beside its closest other (the Qwen3 decoder; "
-                         "for detatar, Puresun; for gibavik, Kobolix; for sagalorn, Gibavik) at equal sizes")
+                         "for detatar, Puresun; for gibavik, Kobolix; for sagalorn, Gibavik; for dokanex, Gibavik and "
+                         "Detatar) at equal sizes")
     ap.add_argument("--size", default=None, help="with --design: this size alone (w2048 or w4096)")
     args = ap.parse_args()
     if args.gpus != 1:

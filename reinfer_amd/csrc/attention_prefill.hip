@@ -329,6 +329,7 @@ flash_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restr
         // a key past the query (masked below) counts as distance 0: its changed score is never used
 #pragma unroll
         for (int j = 0; j < NC; ++j) {
+          if (!((col_mask >> j) & 1)) continue;            // the other workgroup's column tile
           const int q_pos = pos0 + qi[j];
 #pragma unroll
           for (int ks = 0; ks < 2; ++ks)

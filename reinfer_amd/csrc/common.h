@@ -99,12 +99,13 @@ __device__ __forceinline__ float ra_mod_score(float s, float softcap, bool biase
   return s;
 }
 // The same through the hardware's exponential, logarithm and reciprocal (an ulp or two each), for the kernels whose
-// operands are bfloat16: tanh(x) = 1 - 2 / (1 + e^(2x)), the argument bounded so that e^(2x) stays finite.
+// operands are bfloat16: tanh(x) = 1 - 2 / (1 + e^(2x)), which is -1 where the exponential is 0 and 1 where it is infinite
+// (the division written as a product with the hardware's reciprocal: a division proper is ten instructions).
 __device__ __forceinline__ float ra_mod_score_fast(float s, float softcap, float inv_softcap, bool biased, float r1,
                                                    float r2, int dist) {
   if (softcap > 0.f) {
-    const float x = fminf(fmaxf(s * inv_softcap, -15.f), 15.f);
-    s = softcap * (1.f - __fdividef(2.f, 1.f + __expf(2.f * x)));
+    const float e = __builtin_amdgcn_exp2f(s * (inv_softcap * 2.8853900817779268f));
+    s = fmaf(-2.f * softcap, __builtin_amdgcn_rcpf(1.f + e), softcap);
   }
   if (biased) s -= r1 * 0.6931471805599453f * __log2f(fmaf(r2, (float)dist, 1.f));
   return s;

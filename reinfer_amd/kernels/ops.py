@@ -631,6 +631,11 @@ class HipKernels:
         if window > 0:
             # no token reads more than its window (from the tile that holds its first key) and the kept keys' tiles
             max_ctx = min(max_ctx, int(window) + 15 + -(-int(keep) // 16) * 16)
+            if aligned:
+                # nor more than its chunk, of which it sees half on average: the cut is chosen for three quarters of one (any
+                # cut is right for any number of keys). 1 to 32 requests over chunks of 1024: one part of keys a token, and
+                # nothing to merge, takes 8 to 15 us from the chunk's start to its end, several parts 11 to 18
+                max_ctx = min(max_ctx, max(16, 3 * int(window) // 4))
         if chunk is None:
             chunk, max_chunks, waves = self.decode_chunk(n, num_heads, num_kv_heads, head_dim, max_ctx)
         else:

@@ -48,8 +48,11 @@ _OTHER = {"latent_prep": "latent norm + rotation + cache write", "head_linear": 
 class TimedKernels:
     """A kernel set that times every call of the set it wraps."""
 
-    def __init__(self, inner):
+    def __init__(self, inner, attention_shapes: bool = False):
+        """``attention_shapes``: attention is classed by its heads, head size and window, with the bytes of the keys and
+        values its queries see and the flops of their products."""
         self._inner = inner
+        self._attention_shapes = attention_shapes
         self._names: Dict[int, str] = {}
         self._spans: List[Tuple[str, torch.cuda.Event, torch.cuda.Event, int, int]] = []
         self._filler: Optional[torch.Tensor] = None
@@ -64,6 +67,9 @@ class TimedKernels:
         if method in _QK:
             return "head norm + rotation + cache write"
         if method in _ATTN:
+            if self._attention_shapes and method == "attention":
+                window = f", {'chunk' if kwargs.get('aligned') else 'window'} {args[10]}" if args[10] else ""
+                return f"attention {args[6]}/{args[7]} x {args[8]}{window}"
             return "attention"
         if method in _OTHER:
             return _OTHER[method]
@@ -94,11 +100,28 @@ class TimedKernels:
             if isinstance(w, torch.Tensor) and isinstance(args[0], torch.Tensor):
                 nbytes = w.numel() * w.element_size()
                 flops = 2 * args[0].shape[0] * w.numel()
+            if self._attention_shapes and attr == "attention":
+                nbytes, flops = self._attention_work(args, kwargs)
             if attr == "linear_ranges" and out is None:
                 return out                # it declined (the caller runs the whole product next): nothing was launched
             self._spans.append((self._label(attr, args, kwargs), e0, e1, nbytes, flops))
             return out
         return timed_call
+
+    @staticmethod
+    def _attention_work(args, kwargs):
+        """(bytes of the keys and values that the step's queries see, flops of their products) of an ``attention`` call."""
+        q, batch, heads, kv_heads, size, window = args[0], args[5], args[6], args[7], args[8], args[10]
+
+        def first(p: int) -> int:
+            if not window:
+                return 0
+            return p // window * window if kwargs.get("aligned") else max(0, p - window + 1)
+        keys = pairs = 0
+        for n, start in zip(batch.q_lens, batch.starts):
+            keys += start + n - first(start)
+            pairs += sum(p + 1 - first(p) for p in range(start, start + n))
+        return 2 * keys * kv_heads * size * q.element_size(), 4 * pairs * heads * size
 
     def hold_back(self, milliseconds: float, device="cuda:0") -> None:
         """Queue about this much reading of a large buffer, so that the host can queue a whole step

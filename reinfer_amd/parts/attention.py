@@ -43,7 +43,7 @@ import torch
 from .. import kernels
 from ..config.schema import MixerSpec
 from ..weights import MATRIX, VECTOR, ParamDecl
-from .base import KVNeed, LayerCache, NormTarget, split_input
+from .base import KVNeed, LayerCache, NormTarget, project_out, split_input
 from .registry import lookup, register_mixer
 
 
@@ -288,7 +288,7 @@ class GroupedQueryAttention:
         ops.attention(qkv, width, attn, cache.k, cache.v, batch, H, G, D, self.scale, self.window, cache.group,
                       softcap=self.softcap, distance=self.distance, **self._call_options(qkv))
         if self.fused:
-            return self._project_out(ops, attn, resid, emit)
+            return project_out(ops, attn, self.w_o, resid, emit)
         if self.value_inv_freq is not None or self.w_gate is not None:
             gate = None
             if self.w_gate is not None:
@@ -345,22 +345,4 @@ class GroupedQueryAttention:
         attn = torch.empty((T, self.num_heads * self.head_dim), dtype=self.dtype, device=x.device)
         ops.attention(q_rows, q_stride, attn, cache.k, cache.v, batch, self.num_heads,
                       self.num_kv_heads, self.head_dim, self.scale, self.window, cache.group)
-        return self._project_out(ops, attn, resid, emit)
-
-    def _project_out(self, ops, attn, resid, emit: Optional[NormTarget]):
-        T = attn.shape[0]
-        can_add = getattr(ops, "can_accumulate", None)
-        if resid is not None and can_add and can_add(attn, self.w_o):
-            # x += attn . Wo^T in the epilogue, which can also prepare the norm that follows
-            if emit is not None and emit.finished:
-                done = ops.linear_skinny(attn, self.w_o, resid, accumulate=True, finish=emit.finish)
-                return emit if done else None
-            if emit is not None:
-                written = ops.linear_skinny(attn, self.w_o, resid, accumulate=True, emit=emit.emit)
-                emit.ss = emit.ss[:written]          # as many partial sums a row as the kernel that ran has workgroups
-                return emit
-            ops.linear_skinny(attn, self.w_o, resid, accumulate=True)
-            return None
-        out = torch.empty((T, self.spec.hidden), dtype=self.dtype, device=attn.device)
-        ops.linear(attn, self.w_o, out)
-        return out
+        return project_out(ops, attn, self.w_o, resid, emit)

@@ -198,6 +198,26 @@ class ScaledTerms:
     scales: list
 
 
+def project_out(ops, x: torch.Tensor, weight: torch.Tensor, resid: Optional[torch.Tensor], emit: Optional[NormTarget]):
+    """A part's last product x . W^T. Where it can add into the stream ``resid`` it does and None comes back, or ``emit`` if it
+    also prepared the norm that follows; otherwise the product, in the type of ``x``."""
+    can_add = getattr(ops, "can_accumulate", None)
+    if resid is not None and can_add and can_add(x, weight):
+        # resid += x . W^T in the epilogue, which can also prepare the norm that follows
+        if emit is not None and emit.finished:
+            done = ops.linear_skinny(x, weight, resid, accumulate=True, finish=emit.finish)
+            return emit if done else None
+        if emit is not None:
+            written = ops.linear_skinny(x, weight, resid, accumulate=True, emit=emit.emit)
+            emit.ss = emit.ss[:written]          # as many partial sums a row as the kernel that ran has workgroups
+            return emit
+        ops.linear_skinny(x, weight, resid, accumulate=True)
+        return None
+    out = torch.empty((x.shape[0], weight.shape[0]), dtype=x.dtype, device=x.device)
+    ops.linear(x, weight, out)
+    return out
+
+
 def split_input(x):
     """(tensor, row sums or None) of a part's input, plain or :class:`RowScaled`."""
     if isinstance(x, RowScaled):

@@ -31,7 +31,7 @@ import torch
 from .. import kernels
 from ..config.schema import MixerSpec
 from ..weights import VECTOR, ParamDecl
-from .base import KVNeed, LayerCache
+from .base import KVNeed, LayerCache, NormTarget, project_out, split_input
 from .registry import lookup, register_mixer
 
 
@@ -43,6 +43,8 @@ def _round16(n: int) -> int:
 class LatentAttention:
     graph_safe = True       # no host-side state: a decode step with it can be captured
     adds_in_place = True    # forward(..., resid=) may add the output projection into the stream
+    takes_row_scaled = True     # x may be RowScaled: the fused product applies the row factor
+    emits_for_norm = True       # forward(..., emit=) may fill a NormTarget from the output projection
 
     @classmethod
     def declare_params(cls, spec: MixerSpec, prefix: str) -> List[ParamDecl]:
@@ -159,13 +161,18 @@ class LatentAttention:
             self._groups = groups
         return groups
 
-    def forward(self, x, batch, cache: LayerCache, resid: Optional[torch.Tensor] = None):
+    def forward(self, x, batch, cache: LayerCache, resid: Optional[torch.Tensor] = None,
+                emit: Optional[NormTarget] = None):
         ops = kernels.current()
+        x, row_sums = split_input(x)
         T = x.shape[0]
         H, D, Dv, Dp = self.num_heads, self.head_dim, self.value_dim, self.cache_dim
         slots = batch.slots[cache.group] if cache.writes else batch.no_slots
         proj = torch.empty((T, self.proj_width), dtype=self.dtype, device=x.device)
-        ops.linear(x, self.w_in, proj[:, self.in_off:])
+        if row_sums is None:
+            ops.linear(x, self.w_in, proj[:, self.in_off:])
+        else:
+            ops.linear_skinny(x, self.w_in, proj[:, self.in_off:], row_sums=row_sums)
         if self.q_rank:
             # the queries' latent, normed in float over its own width, then up to the heads
             cq = torch.empty((T, self.q_rank), dtype=self.dtype, device=x.device)
@@ -190,10 +197,4 @@ class LatentAttention:
         ops.head_linear(o_lat, Dp, self.w_values, heads, Dv,
                         gate=proj[:, self.gate_off:self.gate_off + self.gate_width] if self.gated else None,
                         gate_per_head=self.head_gate)
-        can_add = getattr(ops, "can_accumulate", None)
-        if resid is not None and can_add and can_add(heads, self.w_o):
-            ops.linear_skinny(heads, self.w_o, resid, accumulate=True)
-            return None
-        out = torch.empty((T, self.spec.hidden), dtype=self.dtype, device=x.device)
-        ops.linear(heads, self.w_o, out)
-        return out
+        return project_out(ops, heads, self.w_o, resid, emit)

@@ -68,9 +68,9 @@ DK_B = {
 # chunks, one that is a multiple and one that is not
 DK_C = {
     "architecture": "Dokanex", "vocab": 257, "width": 96, "norm": {"eps": 1e-4}, "embedding": {"scale": 6.0},
-    "logit_softcap": 30.0,
+    "logit_softcap": 28.0,
     "layers": [attn(8, 1, 32, 32, 16, 15.0, ff=128), attn(8, 1, 32, 32, 48, 15.0, kv_from=0), latent(4, 32, 16, 48, 40, 64,
-               1000000.0, scaling=(8.0, 64, 4.0, 1.0), ff=64), attn(6, 3, 64, 48, 40, 5.0),
+               250000.0, scaling=(6.0, 64, 4.0, 1.0), ff=64), attn(6, 3, 64, 48, 40, 5.0),
                attn(8, 1, 32, 32, 40, kv_from=0), attn(6, 3, 64, 48, 24, kv_from=3, ff=64)],
 }
 # whatever may be absent is absent, the chunks too; no rotation; part of the rotated width turned; a width of 42

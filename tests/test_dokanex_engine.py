@@ -125,7 +125,7 @@ def test_configuration_errors_name_the_key():
 
 def test_the_position_part_has_the_scaled_frequencies():
     for rot in ({"dims": 12, "base": 500.0, "scaling": {"factor": 4.0, "original": 40, "fast": 8.0, "slow": 1.0}},
-                {"dims": 8, "base": 1e6, "scaling": {"factor": 8.0, "original": 2048, "fast": 32.0, "slow": 1.0}},
+                {"dims": 10, "base": 2e5, "scaling": {"factor": 10.0, "original": 1500, "fast": 24.0, "slow": 1.0}},
                 {"dims": 32, "base": 200.0, "scaling": {"factor": 8.0, "original": 1000, "fast": 2.0, "slow": 2.0}},
                 {"dims": 6, "base": 50.0}):
         want, amp = plain.yarn(rot)

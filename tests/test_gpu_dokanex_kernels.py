@@ -110,7 +110,7 @@ def test_attention_plain(dtype, Hq, Hkv, d):
             close(out, ref, 2e-5 if dtype == "float32" else 2 ** -7)
 
 
-@pytest.mark.parametrize("Hq,Hkv,d", [(4, 2, 16), (6, 2, 64), (8, 1, 128), (3, 3, 48), (6, 2, 96), (2, 1, 256)])
+@pytest.mark.parametrize("Hq,Hkv,d", [(4, 2, 16), (6, 2, 64), (8, 1, 128), (3, 3, 48), (10, 2, 80), (9, 3, 112), (2, 1, 256)])
 def test_attention_decode(Hq, Hkv, d):
     ops = kernels.current()
     for bi, (q_lens, starts) in enumerate(DEC_BATCHES[:6]):
@@ -142,7 +142,7 @@ def test_attention_decode_merges_many_parts_of_keys_with_sinks_and_gates():
                 close(out, ref, 2 ** -7)
 
 
-@pytest.mark.parametrize("Hq,Hkv,d", [(4, 2, 16), (6, 2, 64), (8, 1, 128), (3, 3, 48), (6, 2, 96), (2, 1, 256)])
+@pytest.mark.parametrize("Hq,Hkv,d", [(4, 2, 16), (6, 2, 64), (8, 1, 128), (3, 3, 48), (10, 2, 80), (9, 3, 112), (2, 1, 256)])
 def test_attention_prefill(Hq, Hkv, d):
     ops = kernels.current()
     tile = kernels.library.load().ra_attention_prefill_tile(Hq, Hkv, d)
@@ -249,7 +249,7 @@ def test_head_kernel_on_wider_rows_and_on_queries_alone(dtype, Hq, Hkv, d, rot, 
 # ------------------------------------------------------------------ the latent's rotation
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("H,D,R,rank,rot,style,amp", [(3, 20, 12, 40, 12, 1, 1.2), (2, 16, 8, 24, 6, 1, 1.0), (5, 0, 32, 17, 32, 0, 1.4),
-                                                      (4, 64, 16, 128, 16, 1, 0.1 * math.log(8.0) + 1.0), (2, 8, 0, 16, 0, 0, 1.0)])
+                                                      (4, 48, 16, 112, 16, 1, 0.1 * math.log(8.0) + 1.0), (2, 8, 0, 16, 0, 0, 1.0)])
 def test_latent_prep_turns_neighbours_and_takes_a_factor(dtype, H, D, R, rank, rot, style, amp):
     ops = kernels.current()
     torch.manual_seed(rank)

@@ -25,7 +25,7 @@ def draw_config(rng: random.Random, wide: bool = False):
         return rng.choice([None, 1, 2, 5, 16, 17, 33, 64] if not wide else [16, 64, 100, 150, 257])
 
     def cap():
-        return rng.choice([None, 1.5, 6.0, 20.0])
+        return rng.choice([None, 1.5, 6.0, 18.0])
 
     def attention(layers):
         sources = [i for i, L in enumerate(layers) if L["type"] == "attention" and "kv_from" not in L["mixer"]]
@@ -43,7 +43,7 @@ def draw_config(rng: random.Random, wide: bool = False):
     def latents(layers):
         rot = rng.choice([0, 2, 4, 12, 16, 32] if not wide else [16, 32, 64])
         dim = rng.choice([8, 12, 16, 20, 32] if not wide else [48, 64, 128])
-        scaling = (rng.choice([1.0, 2.0, 8.0, 40.0]), rng.choice([16, 100, 2048]), rng.choice([4.0, 32.0]),
+        scaling = (rng.choice([1.0, 2.0, 6.0, 40.0]), rng.choice([16, 100, 3000]), rng.choice([4.0, 32.0]),
                    rng.choice([0.5, 1.0])) if rng.random() < 0.7 else None
         dims = None if rng.random() < 0.7 else rng.choice([r for r in (0, 2, 4, 12, 16) if r <= rot])
         return latent(rng.choice([1, 2, 3, 5, 8, 18] if not wide else [2, 4, 8, 16]), dim, rot, rng.choice([4, 8, 12, 20, 32]),
